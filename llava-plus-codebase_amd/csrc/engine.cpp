@@ -92,7 +92,8 @@ Model::Model(const lmx_config& c) : cfg(c) {
 Model::~Model() {
     if (comm) (void)ncclCommDestroy(comm);
     for (int r = 0; r < P2P_MAX_WORLD; ++r) if (p2p_peer[r] && p2p_peer[r] != p2p_local) (void)hipIpcCloseMemHandle(p2p_peer[r]);
-    if (p2p_local) (void)hipFree(p2p_local);
+    // p2p_local stays allocated until the process ends: uncached device memory that kernels have read must not be freed (tensors allocated after such a free have
+    // held wrong values)
     if (comm_stream) (void)hipStreamDestroy(comm_stream);
     for (auto& r : prof_recs) { (void)hipEventDestroy(r.e0); (void)hipEventDestroy(r.e1); }
     for (auto e : prof_pool) (void)hipEventDestroy(e);

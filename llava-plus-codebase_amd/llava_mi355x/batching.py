@@ -9,7 +9,7 @@ their stop condition, between any two steps.
 
     DecodeBatch     thin wrapper of lmx_batch_* (explicit batched steps: tests, bench, offline batch generation)
     DecodeBatcher   the scheduler (used by LlavaLlamaForCausalLM.generate once enable_batching() was called): the decode thread that steps the live
-                    requests and — packed_prefill, single process — a prefill thread on a high-priority stream that prefills the requests waiting at that
+                    requests and — packed_prefill, single process — a prefill thread on a stream of its own that prefills the requests waiting at that
                     moment TOGETHER (lmx_prefill_batch) beside the running decode steps and hands them over between two steps
 
 Under tensor parallelism (one process per GPU) the scheduler of rank 0 is the LEADER: it is the only thread that issues work carrying
@@ -104,7 +104,7 @@ class DecodeBatcher:
         self.channel = channel          # tensor-parallel leader: tp_serving.CommandChannel to the followers (None: single process)
         self._step_status = None        # tensor parallel: pending ok / fail exchange of the last announced decode step (CommandChannel.agree_begin)
         self.scheduler_prefill = bool(scheduler_prefill) or channel is not None      # requests are prefilled by the scheduler, several at a time
-        # single process: the packed prefills run on a thread and a (high-priority) stream of their own, so a new request neither waits behind the decode
+        # single process: the packed prefills run on a thread and a stream of their own, so a new request neither waits behind the decode
         # step in flight nor holds the live requests' next step back.  Under tensor parallelism every call that carries a collective must
         # be issued in ONE order on every rank: there the prefills stay between two decode steps on the leader's stream
         self.prefill_thread = bool(prefill_thread) and self.scheduler_prefill and channel is None
@@ -487,7 +487,7 @@ class DecodeBatcher:
         try:
             model = self.model
             torch.cuda.set_device(model.device)
-            stream = torch.cuda.Stream(device=model.device, priority=-1)
+            stream = torch.cuda.Stream(device=model.device)
             with torch.cuda.stream(stream):
                 while True:
                     with self._cv:

@@ -887,7 +887,7 @@ class LlavaLlamaForCausalLM:
         granularity.  `max_prefill_rows` bounds the rows of one packed prefill (default 2304: two single-image 512-token requests), i.e. how long the live requests
         wait between two of their decode steps (~18 ms per 1k rows at 7B) and the packed workspace; 0 = up to max_prefill_batch requests whatever
         their size (best burst throughput, unbounded stall).  `prefill_chunk` > 0 bounds the rows per prefill piece (workspace; costs GEMM efficiency).
-        prefill_thread (single process only) = 2 (default): the packed prefills run on their own thread and high-priority stream beside the decode steps instead
+        prefill_thread (single process only) = 2 (default): the packed prefills run on their own thread and stream beside the decode steps instead
         of between two of them — a new request does not wait behind the step in flight, the live requests do not wait for its prefill — and each request's
         rank-local half (image encode / feature-cache hit, splice, prefix-cache take) runs on the request's own thread before it queues; 1 = that half on the
         prefill thread too; 0 = round 4's order (one loop: prefill, then step)."""

@@ -15,7 +15,8 @@ CSRC = os.path.join(ROOT, "llava-plus-codebase_amd", "csrc")
 @pytest.mark.skipif(shutil.which("hipcc") is None and not os.path.exists("/opt/rocm/bin/hipcc"), reason="hipcc not available")
 def test_hot_gemm8p_instantiations_have_no_scratch(tmp_path):
     hipcc = shutil.which("hipcc") or "/opt/rocm/bin/hipcc"
-    r = subprocess.run([hipcc, "-O3", "-std=c++17", "-fPIC", "--offload-arch=gfx950", "-I.", "-I../../include", "-c", "gemm8p.hip", "-o", str(tmp_path / "g.o"),
+    r = subprocess.run([hipcc, "-O3", "-std=c++17", "-fPIC", "--offload-arch=gfx950", "-I.", "-I../../include",
+                        "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops", "-c", "gemm8p.hip", "-o", str(tmp_path / "g.o"),
                         "-Rpass-analysis=kernel-resource-usage"], cwd=CSRC, capture_output=True, text=True, timeout=900)
     assert r.returncode == 0, r.stderr[-2000:]
     usage = {}
