@@ -70,6 +70,39 @@ int lmx_abi_version(void);
 int lmx_create(const lmx_config* cfg, lmx_model** out);
 int lmx_destroy(lmx_model* m);
 
+/* Layer-stack decoders: models described layer by layer on the same sequences, batches, samplers and entry points (lmx_prefill*, lmx_decode*, lmx_seq_*, lmx_batch_*).
+ * Per layer x <- x + m norm1b(attention(norm1 x)), x <- x + m norm2b(mlp(norm2 x)) with RMS norms, an fp32 residual stream and fp32, optionally soft-capped logits.
+ * Layers [loop_start, loop_stop) run loop_times times in a row on the same weights (own caches per pass; the embedding row is added before each pass but the first). */
+typedef struct lmx_layer_config {
+    int32_t n_heads, n_kv_heads, qk_dim, v_dim;
+    float attn_scale;            /* factor on q . k */
+    int32_t window;              /* keys a query sees, itself included (0 = all earlier) */
+    int32_t softmax_sink;        /* 1: the softmax denominator has one more term exp(0) */
+    int32_t qk_norm;             /* 1: RMS norm over qk_dim on every query / key head before the rotation */
+    int32_t qkv_bias;
+    int32_t out_gate;            /* 1: head h's output times sigmoid(W_g x)[h] */
+    int32_t rope_dims;           /* leading dimensions rotated, pairs (i, i + rope_dims / 2); 0 = none */
+    int32_t rope_table;          /* index for lmx_stack_set_rope */
+    int32_t ff;                  /* SiLU-gated feed-forward width, 0 = no feed-forward */
+    int32_t reserved[8];
+} lmx_layer_config;
+typedef struct lmx_stack_config {
+    int32_t abi_version, dtype;
+    int32_t width, vocab_size, n_layers, max_position;
+    int32_t loop_start, loop_stop, loop_times;
+    float norm_eps, residual_mult, logit_softcap;      /* logit_softcap 0 = none */
+    int32_t gemm_variant;
+    int32_t reserved[8];
+} lmx_stack_config;
+int lmx_create_stack(const lmx_stack_config* cfg, const lmx_layer_config* layers, lmx_model** out);
+/* host_cos_sin[p * dims + i] = cos of pair i's angle at position p for i < dims / 2, then the sines */
+int lmx_stack_set_rope(lmx_model* m, int32_t table, int32_t dims, const float* host_cos_sin, int32_t n_pos);
+/* widths of the rows this model exchanges: embedding / residual rows (elements), logit rows (elements), dtype of logits, layer runs (cache slots; rows of a residual trace) */
+int lmx_row_pitch(const lmx_model* m);
+int lmx_vocab_pitch(const lmx_model* m);
+int lmx_logit_dtype(const lmx_model* m);
+int lmx_layer_runs(const lmx_model* m);
+
 /* Copy one checkpoint tensor into the engine (engine-owned, re-laid-out: fused QKV, [32 gate|32 up] interleave, K-padded
  * patch embedding, TP shard selection).  `name` uses HF checkpoint names with the llava prefixes stripped:
  *   model.embed_tokens.weight, model.layers.N.{self_attn.{q,k,v,o}_proj,mlp.{gate,up,down}_proj}.weight,
@@ -385,6 +418,10 @@ int lmx_seq_truncate(lmx_seq* s, int32_t n_rows, void* stream);
  * the rows of all sequences are processed as ONE row block in pieces of block_rows (0 = everything at once), every linear as a single GEMM over
  * the piece; RoPE / KV append / causal attention per sequence against its own cache; each sequence's last row gets the lm_head and its pick
  * (greedy != 0), exactly as lmx_prefill does.  embeds[i]: [n_tokens[i], hidden] rows of request i (output of lmx_gather_embeds). */
+/* The same, with the logits of chosen rows (layer-stack decoders): n_want[i] ascending row indices of sequence i's portion, concatenated in want_rows;
+ * logits_dev receives [sum n_want][vocab pitch] floats. */
+int lmx_prefill_batch_logits(lmx_model* m, lmx_seq* const* seqs, int32_t n, const void* const* embeds, const int32_t* n_tokens, int32_t block_rows, const int32_t* n_want,
+                             const int32_t* want_rows, float* logits_dev, int32_t greedy, void* stream);
 int lmx_prefill_batch(lmx_model* m, lmx_seq* const* seqs, int32_t n, const void* const* embeds, const int32_t* n_tokens, int32_t block_rows, int32_t greedy,
                       void* stream);
 int lmx_op_beam_topk(int32_t dtype, const void* logits, int32_t ld, int32_t V, int32_t rows, const float* beam_scores_dev, int32_t K, float* out_scores, int32_t* out_ids,

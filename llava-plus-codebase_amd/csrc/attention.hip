@@ -29,7 +29,9 @@ namespace lmx {
 // group — whose MFMA and VALU phases interleave.  Tiles are staged in ROUNDS (tile 2r for group 0, 2r + 1 for group 1; each group's four waves DMA
 // their own tile) into a ring of NRND rounds, one workgroup barrier per round.  At the end group 1 hands its (O, m, l) to group 0 through the (then
 // free) ring and group 0 merges the two online-softmax states per lane: m = max(m0, m1), O = O0 2^(m0 - m) + O1 2^(m1 - m), l likewise.
-template <typename T, int D, bool CAUSAL>
+// WIN (FlashArgs::win): sliding window, softmax sink and output gate of the windowed decoders.  Only the key tiles a query block can see are walked: the tile
+// range starts at the tile of the first row's oldest visible key, so the work per block is bounded by the window.
+template <typename T, int D, bool CAUSAL, bool WIN = false>
 __global__ __launch_bounds__(512) void flash_prefill2_kernel(FlashArgs a) {
     constexpr int KSTEPS = D / 16;        // MFMA k-steps over the head dim (QKᵀ)
     constexpr int DB = D / 32;            // 32-row blocks of Oᵀ
@@ -85,7 +87,13 @@ __global__ __launch_bounds__(512) void flash_prefill2_kernel(FlashArgs a) {
         const int lim = a.q_pos0 + (last_q < a.q_len ? last_q : a.q_len - 1) + 1;
         kv_end = lim < kv_end ? lim : kv_end;
     }
-    const int ntiles = (kv_end + FA_KT - 1) / FA_KT;
+    // first tile of the walk (tile indices below are relative to it)
+    int tile0 = 0;
+    if constexpr (WIN) {
+        const int oldest = a.window > 0 ? a.q_pos0 + qb * FA_QB - a.window + 1 : 0;
+        tile0 = oldest > 0 ? oldest / FA_KT : 0;
+    }
+    const int ntiles = (kv_end + FA_KT - 1) / FA_KT - tile0;
 
     f32x16 oacc[DB];
 #pragma unroll
@@ -122,8 +130,8 @@ __global__ __launch_bounds__(512) void flash_prefill2_kernel(FlashArgs a) {
     };
     auto stage = [&](int t, int slot) {
         const unsigned base = lds_base + slot * BUF_BYTES;
-        const T* kt = Kc + (size_t)t * FA_KT * D;
-        const T* vt = Vt + (size_t)t * FA_KT;
+        const T* kt = Kc + (size_t)(tile0 + t) * FA_KT * D;
+        const T* vt = Vt + (size_t)(tile0 + t) * FA_KT;
 #pragma unroll
         for (int i = 0; i < KPPW; ++i) dma(kt + ksrc[i], __builtin_amdgcn_readfirstlane(base + (wave + 4 * i) * 1024));
 #pragma unroll
@@ -167,16 +175,18 @@ __global__ __launch_bounds__(512) void flash_prefill2_kernel(FlashArgs a) {
         // masking only on tiles that can contain an invisible key for some row of this wave (wave-uniform test)
         float p[2][16];
         float tmax = -INFINITY;
-        const int tile_last = t * FA_KT + FA_KT - 1;
-        const bool need_mask = tile_last >= a.kv_len || (CAUSAL && tile_last > a.q_pos0 + q0);
+        const int tile_first = (tile0 + t) * FA_KT, tile_last = tile_first + FA_KT - 1;
+        bool need_mask = tile_last >= a.kv_len || (CAUSAL && tile_last > a.q_pos0 + q0);
+        if constexpr (WIN) need_mask = need_mask || (a.window > 0 && tile_first <= a.q_pos0 + q0 + 31 - a.window);
         if (need_mask) {
 #pragma unroll
             for (int kb = 0; kb < 2; ++kb)
 #pragma unroll
                 for (int r = 0; r < 16; ++r) {
-                    const int key = t * FA_KT + kb * 32 + (r & 3) + 4 * ((r >> 2) & 1) + 8 * hi + 16 * (r >> 3);
+                    const int key = tile_first + kb * 32 + (r & 3) + 4 * ((r >> 2) & 1) + 8 * hi + 16 * (r >> 3);
                     bool ok = key < a.kv_len;
                     if (CAUSAL) ok = ok && (key <= my_pos);
+                    if constexpr (WIN) ok = ok && (a.window <= 0 || my_pos - key < a.window);
                     const float v = ok ? sacc[kb][r] * sc : -INFINITY;
                     p[kb][r] = v;
                     tmax = fmaxf(tmax, v);
@@ -269,7 +279,17 @@ __global__ __launch_bounds__(512) void flash_prefill2_kernel(FlashArgs a) {
             for (int r = 0; r < 16; ++r) oacc[i][r] = oacc[i][r] * a0 + mg[(i * 16 + r) * 64 + lane] * a1;
     }
     const float l_tot = l_run + __shfl_xor(l_run, 32, 64);
-    const float inv = l_tot > 0.f ? 1.f / l_tot : 0.f;
+    float inv = l_tot > 0.f ? 1.f / l_tot : 0.f;
+    if constexpr (WIN) {
+        if (a.sink) {                          // the running maximum may lie below the sink's score 0: bring both sums to max(m, 0)
+            const float m2 = fmaxf(m_run, 0.f), f = __builtin_amdgcn_exp2f(m_run - m2);
+            inv = f / (l_tot * f + __builtin_amdgcn_exp2f(-m2));
+        }
+        if (a.gate && qrow < a.q_len) {
+            const float g = to_f32(reinterpret_cast<const T*>(a.gate)[(size_t)qrow * a.q_stride + head]);
+            inv *= 1.f / (1.f + __expf(-g));
+        }
+    }
     if (a.lse && hi == 0 && qrow < a.q_len) a.lse[(size_t)head * a.lse_stride + qrow] = m_run + __builtin_amdgcn_logf(l_tot);      // v_log_f32 = log2
     if (qrow < a.q_len) {
         T* op = reinterpret_cast<T*>(a.O) + (size_t)qrow * a.o_stride + head * D;
@@ -296,9 +316,10 @@ void launch_flash_prefill(int dtype, int D, const FlashArgs& a, hipStream_t st) 
     {
         // two key groups per query block (flash_prefill2_kernel): 8 waves, ring of 2 (D = 128) / 3 (D = 64) rounds of two tiles
         const int smem2 = (D == 128 ? 2 : 3) * 2 * (FA_KT * D * 2 + D * FA_KT * 2);
-#define LMX_FA2_LAUNCH(TT, DD, CC)                                                                                  \
+#define LMX_FA2_LAUNCH(TT, DD, CC) LMX_FA2_LAUNCH_W(TT, DD, CC, false)
+#define LMX_FA2_LAUNCH_W(TT, DD, CC, WW)                                                                            \
     do {                                                                                                            \
-        auto kern = flash_prefill2_kernel<TT, DD, CC>;                                                              \
+        auto kern = flash_prefill2_kernel<TT, DD, CC, WW>;                                                            \
         static bool attr_set = false;                                                                               \
         if (!attr_set) {                                                                                            \
             LMX_CHECK_HIP(hipFuncSetAttribute(reinterpret_cast<const void*>(kern), hipFuncAttributeMaxDynamicSharedMemorySize, smem2)); \
@@ -306,7 +327,11 @@ void launch_flash_prefill(int dtype, int D, const FlashArgs& a, hipStream_t st) 
         }                                                                                                           \
         hipLaunchKernelGGL(kern, grid, dim3(512), smem2, st, a);                                                    \
     } while (0)
-        if (dtype == kBF16) {
+        if (a.win) {
+            LMX_REQUIRE(a.causal && !a.lse, "flash prefill: the windowed form is causal and keeps no log-sum-exp");
+            if (dtype == kBF16) { if (D == 128) LMX_FA2_LAUNCH_W(bf16_t, 128, true, true); else LMX_FA2_LAUNCH_W(bf16_t, 64, true, true); }
+            else { if (D == 128) LMX_FA2_LAUNCH_W(f16_t, 128, true, true); else LMX_FA2_LAUNCH_W(f16_t, 64, true, true); }
+        } else if (dtype == kBF16) {
             if (D == 128) { if (a.causal) LMX_FA2_LAUNCH(bf16_t, 128, true); else LMX_FA2_LAUNCH(bf16_t, 128, false); }
             else          { if (a.causal) LMX_FA2_LAUNCH(bf16_t, 64, true);  else LMX_FA2_LAUNCH(bf16_t, 64, false); }
         } else {
@@ -314,6 +339,7 @@ void launch_flash_prefill(int dtype, int D, const FlashArgs& a, hipStream_t st) 
             else          { if (a.causal) LMX_FA2_LAUNCH(f16_t, 64, true);  else LMX_FA2_LAUNCH(f16_t, 64, false); }
         }
 #undef LMX_FA2_LAUNCH
+#undef LMX_FA2_LAUNCH_W
         LMX_CHECK_HIP(hipGetLastError());
         return;
     }

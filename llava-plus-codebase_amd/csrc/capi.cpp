@@ -10,7 +10,7 @@
 
 using namespace lmx;
 
-struct lmx_model { Model impl; explicit lmx_model(const lmx_config& c) : impl(c) {} };
+struct lmx_model { Model impl; explicit lmx_model(const lmx_config& c) : impl(c) {} lmx_model(const lmx_stack_config& c, const lmx_layer_config* l) : impl(c, l) {} };
 struct lmx_seq { Seq impl; explicit lmx_seq(Model* m) : impl(m) {} };
 struct lmx_batch { Batch impl; lmx_batch(Model* m, int cap) : impl(m, cap) {} };
 
@@ -37,6 +37,25 @@ int lmx_create(const lmx_config* cfg, lmx_model** out) {
     *out = new lmx_model(*cfg);
     LMX_API_END
 }
+int lmx_create_stack(const lmx_stack_config* cfg, const lmx_layer_config* layers, lmx_model** out) {
+    LMX_API_BEGIN
+    LMX_REQUIRE(cfg && layers && out, "lmx_create_stack: null argument");
+    int n = 0;
+    LMX_CHECK_HIP(hipGetDeviceCount(&n));
+    LMX_REQUIRE(n > 0, "no HIP device visible");
+    *out = new lmx_model(*cfg, layers);
+    LMX_API_END
+}
+int lmx_stack_set_rope(lmx_model* m, int32_t table, int32_t dims, const float* host_cos_sin, int32_t n_pos) {
+    LMX_API_BEGIN
+    LMX_REQUIRE(m, "null model");
+    m->impl.stack_set_rope(table, dims, host_cos_sin, n_pos);
+    LMX_API_END
+}
+int lmx_row_pitch(const lmx_model* m) { return m ? m->impl.H : -1; }
+int lmx_vocab_pitch(const lmx_model* m) { return m ? m->impl.V : -1; }
+int lmx_logit_dtype(const lmx_model* m) { return m ? m->impl.logit_dtype() : -1; }
+int lmx_layer_runs(const lmx_model* m) { return m ? m->impl.L : -1; }
 int lmx_destroy(lmx_model* m) {
     LMX_API_BEGIN
     if (m) {
@@ -691,6 +710,29 @@ int lmx_prefill_batch(lmx_model* m, lmx_seq* const* seqs, int32_t n, const void*
     std::vector<Seq*> ss((size_t)n);
     for (int i = 0; i < n; ++i) { LMX_REQUIRE(seqs[i] != nullptr, "null sequence"); ss[(size_t)i] = &seqs[i]->impl; }
     m->impl.prefill_multi(ss.data(), embeds, n_tokens, n, block_rows, greedy != 0, S(stream));
+    LMX_API_END
+}
+int lmx_prefill_batch_logits(lmx_model* m, lmx_seq* const* seqs, int32_t n, const void* const* embeds, const int32_t* n_tokens, int32_t block_rows, const int32_t* n_want,
+                             const int32_t* want_rows, float* logits_dev, int32_t greedy, void* stream) {
+    LMX_API_BEGIN
+    LMX_REQUIRE(m && seqs && embeds && n_tokens && n >= 1 && n_want, "null argument");
+    LMX_REQUIRE(m->impl.stk, "prefill_batch_logits: layer-stack decoders only (fp32 logits)");
+    std::vector<Seq*> ss((size_t)n);
+    std::vector<std::vector<int>> want((size_t)n);
+    size_t off = 0;
+    for (int i = 0; i < n; ++i) {
+        LMX_REQUIRE(seqs[i] != nullptr && n_want[i] >= 0 && (n_want[i] == 0 || (want_rows && logits_dev)), "prefill_batch_logits: bad sequence or rows");
+        ss[(size_t)i] = &seqs[i]->impl;
+        for (int k = 0; k < n_want[i]; ++k) {
+            const int r = want_rows[off + (size_t)k];
+            LMX_REQUIRE(r >= 0 && r < n_tokens[i] && (k == 0 || r > want[(size_t)i].back()), "prefill_batch_logits: wanted rows must ascend inside the portion");
+            want[(size_t)i].push_back(r);
+        }
+        off += (size_t)n_want[i];
+    }
+    StackOutputs o;
+    o.logits = off ? logits_dev : nullptr; o.want = want.data();
+    m->impl.stack_prefill(ss.data(), embeds, n_tokens, n, block_rows, greedy != 0, o, S(stream));
     LMX_API_END
 }
 int lmx_seq_copy(lmx_seq* dst, const lmx_seq* src, void* stream) {

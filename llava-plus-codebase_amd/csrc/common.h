@@ -167,6 +167,9 @@ __device__ __forceinline__ float act_quick_gelu(float x) { return x / (1.f + __e
 __device__ __forceinline__ float act_gelu_erf(float x) { return 0.5f * x * (1.f + erff(x * 0.70710678118654752f)); }
 __device__ __forceinline__ float act_silu(float x) { return x / (1.f + __expf(-x)); }
 
+// logits <- cap tanh(logits / cap); cap <= 0: unchanged
+__device__ __forceinline__ float soft_cap(float v, float cap) { return cap > 0.f ? cap * tanhf(v / cap) : v; }
+
 // ---- XCD-aware block remap (8 XCDs, block b is dispatched to XCD b % 8). Bijective for any nwg.
 __device__ __forceinline__ int xcd_remap(int bid, int nwg) {
     const int xcd = bid & 7, idx = bid >> 3;

@@ -41,7 +41,7 @@ Model::Model(const lmx_config& c) : cfg(c) {
     LMX_REQUIRE(c.abi_version == LMX_ABI_VERSION, "lmx_config.abi_version mismatch");
     LMX_REQUIRE(c.dtype == kF32 || c.dtype == kBF16 || c.dtype == kF16, "bad dtype");
     LMX_REQUIRE(c.tp_world >= 1 && c.tp_rank >= 0 && c.tp_rank < c.tp_world, "bad tensor-parallel rank/world");
-    es = (int)dtype_size(c.dtype);
+    es = les = (int)dtype_size(c.dtype);
     // defaults of the options lmx_model_set_option can flip later (A/B runs and the bit-identity tests of the fused forms)
     { const char* e = getenv("LMX_FUSE_ROPE"); if (e) opt_fuse_rope = atoi(e) != 0; }
     { const char* e = getenv("LMX_VIS_PACK"); if (e) opt_vis_pack = atoi(e) != 0; }
@@ -138,6 +138,7 @@ static void copy_block(void* dst, int dst_cols, int dst_row0, const void* src, i
 void Model::load_weight(const std::string& name, const void* src, int dtype, int ndim, const int64_t* shape, hipStream_t st) {
     LMX_REQUIRE(dtype == cfg.dtype, "weight dtype must equal the model dtype (cast on the host side): " + name);
     LMX_REQUIRE(src != nullptr && ndim >= 1 && ndim <= 4, "bad tensor: " + name);
+    if (stk) { stack_load_weight(name, src, ndim, shape, st); return; }
     int64_t numel = 1;
     for (int i = 0; i < ndim; ++i) numel *= shape[i];
     auto expect = [&](std::initializer_list<int64_t> want) {
@@ -264,6 +265,7 @@ void Model::load_weight(const std::string& name, const void* src, int dtype, int
 }
 
 void Model::finalize() {
+    if (stk) { stack_finalize(); return; }
     std::string missing;
     auto need = [&](const std::string& n) { if (!loaded.count(n)) missing += n + " "; };
     need("model.embed_tokens.weight"); need("model.norm.weight"); need("lm_head.weight");
@@ -519,8 +521,9 @@ uint64_t next_seq_uid() { return g_seq_uid.fetch_add(1); }
 Seq::Seq(Model* mm) : m(mm) {
     uid = g_seq_uid.fetch_add(1);
     layer_stride = (size_t)m->nkv_l * m->s_max * m->D * m->es;
-    kc.ensure(layer_stride * m->L, true);
-    vt.ensure(layer_stride * m->L, true);
+    const size_t kv_bytes = m->stk ? m->stk->kv_bytes : layer_stride * m->L;
+    kc.ensure(kv_bytes, true);
+    vt.ensure(kv_bytes, true);
     log_cap = m->s_max + 8;
     state.ensure(16 + (size_t)log_cap * 8, true);
     d_len = state.as<int>(); d_nout = d_len + 1;
@@ -531,16 +534,18 @@ Seq::Seq(Model* mm) : m(mm) {
     // decode workspace
     const int es = m->es;
     n_split = (m->s_max + 127) / 128;          // fixed 128-key chunks (attention.hip: DF_CHUNK)
-    const size_t aws = decode_fused_ws_floats(m->nh_l, n_split, m->D);
+    const size_t aws = m->stk ? m->stk->dec_ws : decode_fused_ws_floats(m->nh_l, n_split, m->D);
     size_t off = 0;
     auto carve = [&](size_t bytes) { size_t o = off; off += (bytes + 255) / 256 * 256; return o; };
     const size_t o_h = carve((size_t)m->H * es), o_qkv = carve((size_t)m->qkv_n * es), o_attn = carve((size_t)m->nh_l * m->D * es),
-                 o_act = carve((size_t)m->I_l * es), o_log = carve((size_t)m->V * es), o_aws = carve(aws * 4), o_cnt = carve((size_t)m->nh_l * 4);
+                 o_act = carve((size_t)m->I_l * es), o_log = carve((size_t)m->V * m->les), o_aws = carve(aws * 4), o_cnt = carve((size_t)m->nh_l * 4);
+    const size_t o_x = m->stk ? carve((size_t)m->H * es) : 0, o_y = m->stk ? carve((size_t)m->H * es) : 0, o_xr = m->stk ? carve((size_t)m->H * 8) : 0;
     dws.ensure(off, true);
     char* W = dws.as<char>();
     d_h = W + o_h; d_qkv = W + o_qkv; d_attn = W + o_attn; d_act = W + o_act; d_logits = W + o_log;
     d_aws = reinterpret_cast<float*>(W + o_aws);
     d_cnt = reinterpret_cast<int*>(W + o_cnt);
+    if (m->stk) { d_x = W + o_x; d_y = W + o_y; d_xr = reinterpret_cast<float*>(W + o_xr); }
     kv_gran.ensure((size_t)2 * m->nkv_l * m->D * 8, true);
     LMX_CHECK_HIP(hipHostMalloc(reinterpret_cast<void**>(&h_status), sizeof(unsigned), hipHostMallocMapped));
     *h_status = 0;
@@ -558,6 +563,14 @@ Seq::~Seq() {
 // ---------------------------------------------------------------------------------------------------------------
 void Model::prefill(Seq* s, const void* embeds, int T, int chunk, void* logits, bool logits_all, bool greedy, hipStream_t st, void* hidden, void* attn_probs) {
     LMX_REQUIRE(T > 0 && embeds, "prefill: empty input");
+    if (stk) {
+        LMX_REQUIRE(!attn_probs, "output_attentions: not available for a layer-stack decoder");
+        StackOutputs o;
+        if (logits_all) o.logits = static_cast<float*>(logits); else o.last_logits = static_cast<float*>(logits);
+        o.hidden = static_cast<float*>(hidden);
+        stack_prefill(&s, &embeds, &T, 1, chunk, greedy, o, st);
+        return;
+    }
     LMX_REQUIRE(!attn_probs || (cfg.tp_world == 1 && comm == nullptr), "output_attentions: single process only (a tensor-parallel rank holds a slice of the heads)");
     const int kv_after = s->len + T;                        // key range of the attention maps' rows: [0, len + T)
     LMX_REQUIRE(s->len + T <= s_max, "prefill: sequence would exceed the KV-cache capacity (max_position)");
@@ -717,6 +730,7 @@ void Model::prefill(Seq* s, const void* embeds, int T, int chunk, void* logits, 
 // order of their fp32 partial sums).  Each sequence's last row goes through the lm_head and its pick, exactly as Model::prefill does.
 void Model::prefill_multi(Seq* const* seqs, const void* const* embeds, const int* Ts, int n, int block_rows, bool greedy, hipStream_t st) {
     LMX_REQUIRE(n >= 1 && seqs && embeds && Ts, "prefill_multi: bad arguments");
+    if (stk) { stack_prefill(seqs, embeds, Ts, n, block_rows, greedy, StackOutputs{}, st); return; }
     LMX_REQUIRE(rope != nullptr, "rope table not set");
     long total = 0;
     for (int i = 0; i < n; ++i) {
@@ -822,6 +836,7 @@ void Seq::check_wait_status(hipStream_t st) {
 // llava_arch.py:103-112).  16-bit models take the split-q form (decode_attn.hip): q alone, then ONE launch holding the attention workgroups and the k|v
 // projection, so that the attention's latency chain runs under the k|v weight stream — bit-identical to the three-launch form.
 void Model::decode_step_launch(Seq* s, hipStream_t st, int64_t* id_out) {
+    if (stk) { stack_decode_step(s, st, id_out); return; }
     const int dt = cfg.dtype;
     const bool lead = cfg.tp_rank == 0;
     const float scale = 1.f / sqrtf((float)D);
@@ -875,9 +890,12 @@ void Model::seq_copy(Seq* dst, const Seq* src, hipStream_t st) {
     LMX_REQUIRE(dst && src && dst->m == this && src->m == this && dst != src, "seq_copy: bad sequences");
     LMX_REQUIRE(src->len > 0, "seq_copy: the source has no context");
     const size_t n = (size_t)src->len;
+    if (stk) stack_seq_copy(dst, src, st);
+    else {
     // K rows [L][kv_head][s_max][D]: n * D contiguous elements per (layer, head);  V^T [L][kv_head][D][s_max]: n contiguous elements per (layer, head, d)
     LMX_CHECK_HIP(hipMemcpy2DAsync(dst->kc.p, (size_t)s_max * D * es, src->kc.p, (size_t)s_max * D * es, n * D * es, (size_t)L * nkv_l, hipMemcpyDeviceToDevice, st));
     LMX_CHECK_HIP(hipMemcpy2DAsync(dst->vt.p, (size_t)s_max * es, src->vt.p, (size_t)s_max * es, n * es, (size_t)L * nkv_l * D, hipMemcpyDeviceToDevice, st));
+    }
     dst->len = src->len;
     launch_set_state(dst->d_len, dst->len, dst->d_tok, 0, 0, dst->d_nout, 0, st);
     dst->last_stream = st; dst->used = true;
@@ -899,7 +917,7 @@ void Model::decode(Seq* s, int64_t token, int n_steps, void* logits, bool greedy
         decode_step_launch(s, st);
         s->len += 1;
     }
-    if (logits) LMX_CHECK_HIP(hipMemcpyAsync(logits, s->d_logits, (size_t)V * es, hipMemcpyDeviceToDevice, st));
+    if (logits) LMX_CHECK_HIP(hipMemcpyAsync(logits, s->d_logits, (size_t)V * les, hipMemcpyDeviceToDevice, st));
 }
 
 // ---------------------------------------------------------------------------------------------------------------
@@ -915,6 +933,7 @@ void Model::ensure_batch_weights(hipStream_t st) {
     batch_weights_ready = true;
     const char* e = getenv("LMX_BATCH_SWIZZLE");
     if (cfg.dtype == kF32 || (e && atoi(e) == 0)) return;
+    if (stk) { stack_batch_weights(st); return; }
     auto mk = [&](const void* W, int N, int K) -> void* {
         if (!W) return nullptr;
         void* d = alloc_weight(skinny_swizzled_bytes(N, K, es));
@@ -937,10 +956,12 @@ Batch::Batch(Model* mm, int capacity) : m(mm), cap(capacity) {
     size_t off = 0;
     auto carve = [&](size_t bytes) { size_t o = off; off += (bytes + 255) / 256 * 256; return o; };
     const size_t o_h = carve((size_t)cap * m->H * es), o_x = carve((size_t)cap * m->H * es), o_qkv = carve((size_t)cap * m->qkv_n * es),
-                 o_attn = carve((size_t)cap * m->nh_l * m->D * es), o_act = carve((size_t)cap * m->I_l * es), o_log = carve((size_t)cap * m->V * es);
+                 o_attn = carve((size_t)cap * m->nh_l * m->D * es), o_act = carve((size_t)cap * m->I_l * es), o_log = carve((size_t)cap * m->V * m->les);
+    const size_t o_y = m->stk ? carve((size_t)cap * m->H * es) : 0, o_xr = m->stk ? carve((size_t)cap * m->H * 4) : 0;
     ws.ensure(off, true);
     char* W = ws.as<char>();
     h = W + o_h; x = W + o_x; qkv = W + o_qkv; attn = W + o_attn; act = W + o_act; logits = W + o_log;
+    if (m->stk) { y = W + o_y; xr = reinterpret_cast<float*>(W + o_xr); }
     const size_t attn_bytes = sizeof(DecodeFusedSeq) * (size_t)m->L * cap, state_bytes = sizeof(SeqStateRef) * (size_t)cap;
     tab.ensure(attn_bytes + state_bytes, true);
     if (m->cfg.dtype != kF32) {                     // K-sliced linears of a decode batch: o_proj / down_proj (N = H) and q|k|v
@@ -962,9 +983,10 @@ void Batch::bind(Seq* const* seqs, int n, hipStream_t st) {
     SeqStateRef* stt = reinterpret_cast<SeqStateRef*>(host_tab.data() + sizeof(DecodeFusedSeq) * (size_t)L * cap);
     for (int i = 0; i < n; ++i) {
         Seq* s = seqs[i];
-        for (int l = 0; l < L; ++l)
-            at[(size_t)l * cap + i] = DecodeFusedSeq{s->kc.as<char>() + (size_t)l * s->layer_stride, s->vt.as<char>() + (size_t)l * s->layer_stride,
-                                                     s->d_len, s->d_aws, s->d_cnt};
+        for (int l = 0; l < L; ++l) {
+            const size_t off = m->stk ? m->stk->runs[(size_t)l].kv_off : (size_t)l * s->layer_stride;
+            at[(size_t)l * cap + i] = DecodeFusedSeq{s->kc.as<char>() + off, s->vt.as<char>() + off, s->d_len, s->d_aws, s->d_cnt};
+        }
         stt[i] = SeqStateRef{s->d_len, s->d_nout, s->d_tok, s->d_log, s->log_cap, 0, s->samp, s->d_stop};
     }
     // the previous step's kernels may still be reading the old tables on this stream, and the host image is reused
@@ -1021,10 +1043,15 @@ void Model::decode_batch(Batch* b, Seq* const* seqs, int n, const int64_t* token
             decode_step_launch(s, st, d_ids + (size_t)step * b->cap);      // a lone member reports -1 after a device-side stop exactly like the members of a larger batch
             s->len += 1;
         }
-        if (logits) LMX_CHECK_HIP(hipMemcpyAsync(logits, s->d_logits, (size_t)V * es, hipMemcpyDeviceToDevice, st));
+        if (logits) LMX_CHECK_HIP(hipMemcpyAsync(logits, s->d_logits, (size_t)V * les, hipMemcpyDeviceToDevice, st));
     } else {
     { LMX_PROF("decode_batch.embed"); launch_gather_tokens_batch(dt, b->d_state_tab, n, embed, b->h, H, V, st); }
     for (int step = 0; step < n_steps; ++step) {
+        if (stk) {
+            stack_decode_batch_step(b, seqs, n, d_ids + (size_t)step * b->cap, st);
+            for (int i = 0; i < n; ++i) seqs[i]->len += 1;
+            continue;
+        }
         bool x_ready = false;          // b->x already holds the normalised rows of the NEXT linear (written by the tensor-parallel all-reduce's launch: allreduce_norm)
         for (int l = 0; l < L; ++l) {
             const DecLayerW& w = dec[l];
@@ -1052,7 +1079,7 @@ void Model::decode_batch(Batch* b, Seq* const* seqs, int n, const int64_t* token
         for (int i = 0; i < n; ++i) seqs[i]->len += 1;
     }
     }
-    if (logits && n > 1) LMX_CHECK_HIP(hipMemcpyAsync(logits, b->logits, (size_t)n * V * es, hipMemcpyDeviceToDevice, st));
+    if (logits && n > 1) LMX_CHECK_HIP(hipMemcpyAsync(logits, b->logits, (size_t)n * V * les, hipMemcpyDeviceToDevice, st));
     if (ids_out_host) {       // [n_steps][n], after the stream drained
         LMX_CHECK_HIP(hipMemcpy2DAsync(ids_out_host, (size_t)n * 8, d_ids, (size_t)b->cap * 8, (size_t)n * 8, (size_t)n_steps, hipMemcpyDeviceToHost, st));
         if (sync_ids) {

@@ -4,6 +4,8 @@
 #include <hip/hip_runtime.h>
 #include <rccl/rccl.h>
 #include <map>
+#include <memory>
+#include <algorithm>
 #include <atomic>
 #include <mutex>
 #include <set>
@@ -48,11 +50,38 @@ struct VisLayerW {
     void *ln1w = nullptr, *ln1b = nullptr, *ln2w = nullptr, *ln2b = nullptr;
 };
 
+// ---- layer-stack decoders (stack.cpp) ---------------------------------------------------------------------------------------------------------------------
+struct StackLayer {
+    lmx_layer_config c{};
+    int D = 0, qkv_n = 0, ff = 0, gate_off = -1;         // padded head width, rows of the fused q | k | v | gate weight, padded ff (0: none), first gate row (-1: none)
+    void *wqkv = nullptr, *bqkv = nullptr, *wo = nullptr, *wgu = nullptr, *wd = nullptr, *n1 = nullptr, *n1b = nullptr, *n2 = nullptr, *n2b = nullptr, *qn = nullptr, *kn = nullptr;
+    void *sw_qkv = nullptr, *sw_o = nullptr, *sw_gu = nullptr, *sw_d = nullptr;
+};
+struct StackRun { int layer; bool inject; size_t kv_off; };      // one execution of a layer: own slice of the K and V^T caches (byte offset, same in both)
+struct Stack {
+    lmx_stack_config c{};
+    std::vector<StackLayer> layers;
+    std::vector<StackRun> runs;
+    size_t kv_bytes = 0, dec_ws = 0;                     // bytes of one sequence's K (= V^T) cache; floats of its decode partials
+    int attn_n = 0;                                      // widest concatenation of heads
+    std::vector<float*> rope; std::vector<int> rope_dims;
+    ~Stack() { for (float* p : rope) if (p) (void)hipFree(p); }
+};
+struct StackOutputs {
+    float* logits = nullptr;                             // rows [wanted][V] in the order of the sequences and of `want`
+    const std::vector<int>* want = nullptr;              // per sequence: wanted rows, ascending (null: every row)
+    float* last_logits = nullptr;                        // [n][V]: the last row of each sequence
+    float* hidden = nullptr;                             // one sequence: [runs][T][H] residual stream after every run
+};
+
 struct Seq;
+struct Batch;
 
 struct Model {
     lmx_config cfg{};
     int es = 2;                 // element size
+    int les = 0;                // logit element size: es, or 4 where logits stay in 32 bits (layer-stack decoders)
+    std::unique_ptr<Stack> stk; // set: a layer-stack decoder instead of the LLaMA decoder
     // decoder geometry (TP-local)
     int H = 0, I_l = 0, I_sh = 0, nh_l = 0, nkv_l = 0, D = 0, V = 0, L = 0, qkv_n = 0, s_max = 0;
     int V_l = 0, v_off = 0;     // lm_head rows held by this rank (vocabulary-parallel head under TP) and the id of its first row
@@ -113,6 +142,8 @@ struct Model {
     hipEvent_t vws_done = nullptr; hipStream_t vws_stream = nullptr;
 
     explicit Model(const lmx_config& c);
+    Model(const lmx_stack_config& c, const lmx_layer_config* layers);
+    int logit_dtype() const { return les == 4 ? (int)kF32 : cfg.dtype; }
     ~Model();
     void* alloc_weight(size_t bytes, bool zero = false);
     void load_weight(const std::string& name, const void* src, int dtype, int ndim, const int64_t* shape, hipStream_t st);
@@ -138,6 +169,15 @@ struct Model {
     void seq_copy(Seq* dst, const Seq* src, hipStream_t st);      // dst := src's context (KV of the first src->len positions, length): beam reordering
     void decode_batch(struct Batch* b, Seq* const* seqs, int n, const int64_t* tokens, int n_steps, void* logits, bool greedy, int64_t* ids_out_host, hipStream_t st,
                       bool sync_ids = true);
+    // layer-stack decoders (stack.cpp)
+    void stack_set_rope(int table, int dims, const float* host, int n_pos);
+    void stack_load_weight(const std::string& name, const void* src, int ndim, const int64_t* shape, hipStream_t st);
+    void stack_finalize();
+    void stack_batch_weights(hipStream_t st);
+    void stack_prefill(Seq* const* seqs, const void* const* embeds, const int* Ts, int n, int block_rows, bool greedy, const StackOutputs& out, hipStream_t st);
+    void stack_decode_step(Seq* s, hipStream_t st, int64_t* id_out);
+    void stack_decode_batch_step(struct Batch* b, Seq* const* seqs, int n, int64_t* ids, hipStream_t st);
+    void stack_seq_copy(Seq* dst, const Seq* src, hipStream_t st);
     // ---- options a caller may flip on a live model (lmx_model_set_option; defaults from the environment at creation) ----------------------------------
     // fuse_rope: RoPE + KV append in the prefill's q|k|v GEMM epilogue (gemm8p.hip qkv_rope_epilogue) instead of a rope_kv launch — bit-identical, faster
     // vis_pack:  CLIP K / V^T pack in the tower's q|k|v GEMM epilogue instead of a pack launch — bit-identical, launch count
@@ -179,6 +219,7 @@ struct Seq {
     DevBuf skw;                        // split-K partial tiles of the ping-pong GEMM (o_proj, down_proj of a prefill)
     DevBuf dws;                        // decode workspace
     void *d_h = nullptr, *d_qkv = nullptr, *d_attn = nullptr, *d_act = nullptr, *d_logits = nullptr; float* d_aws = nullptr; int* d_cnt = nullptr;
+    void *d_x = nullptr, *d_y = nullptr; float* d_xr = nullptr;       // layer-stack decoders: normed row, sublayer output, fp32 residual (two rows)
     int n_split = 8;
     DevBuf kv_gran;                    // split-q decode step: {bits, tag} granules [2 nkv_l D] of the newest key / value (zeroed at creation: tag 0 is never used)
     unsigned attn_tag = 1;             // tag of the next split-q launch on kv_gran
@@ -200,6 +241,7 @@ struct Batch {
     int cap = 0;
     DevBuf ws;                         // h | x (normed) | qkv | attn | act | logits, each [cap][...]
     void *h = nullptr, *x = nullptr, *qkv = nullptr, *attn = nullptr, *act = nullptr, *logits = nullptr;
+    void* y = nullptr; float* xr = nullptr;      // layer-stack decoders: sublayer outputs, fp32 residual rows
     DevBuf tab;                        // device: DecodeFusedSeq[L][cap] then SeqStateRef[cap]
     DecodeFusedSeq* d_attn_tab = nullptr; SeqStateRef* d_state_tab = nullptr;
     std::vector<uint64_t> members;     // Seq::uid of what the device tables currently describe

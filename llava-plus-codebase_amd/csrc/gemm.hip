@@ -27,7 +27,7 @@
 
 namespace lmx {
 
-template <typename T, int BM, int BN, int WM, int WN, bool GLDS>
+template <typename T, int BM, int BN, int WM, int WN, bool GLDS, bool F32 = false>
 __global__ __launch_bounds__(WM * WN * 64) void gemm_mfma_kernel(GemmArgs a) {
     constexpr int NW = WM * WN;
     constexpr int NT_ = NW * 64;
@@ -148,7 +148,7 @@ __global__ __launch_bounds__(WM * WN * 64) void gemm_mfma_kernel(GemmArgs a) {
         }
     }
 
-    gemm_epilogue<T, MT, NTL>(a, acc, m0 + wm * TM, n0 + wn * TN, l31, hi);
+    gemm_epilogue<T, MT, NTL, F32>(a, acc, m0 + wm * TM, n0 + wn * TN, l31, hi);
 }
 
 // ---------------------------------------------------------------------------------------------
@@ -397,6 +397,7 @@ __global__ __launch_bounds__(256) void gemm_f32_kernel(GemmArgs a) {
             }
             v = apply_act(v, act);
             if (R) v += R[(size_t)m * a.ldr + n];
+            if (a.c_f32) v = soft_cap(v, a.cap);
             C[(size_t)m * a.ldc + n] = v;
         }
     }
@@ -613,7 +614,8 @@ __global__ __launch_bounds__(256) void gemv_kernel(GemvArgs a) {
             if (bias) v += to_f32(bias[n]);
             v = apply_act(v, a.act);
             if (Rr) v += to_f32(Rr[(size_t)mb * a.ldr + n]);
-            C[(size_t)mb * a.ldc + n] = from_f32<T>(v);
+            if (a.c_f32) reinterpret_cast<float*>(a.C)[(size_t)mb * a.ldc + n] = soft_cap(v, a.cap);
+            else C[(size_t)mb * a.ldc + n] = from_f32<T>(v);
         }
     }
 }
@@ -631,10 +633,10 @@ __global__ __launch_bounds__(256) void gemv2_kernel(GemvArgs a) {
 // ---------------------------------------------------------------------------------------------
 // host launchers
 // ---------------------------------------------------------------------------------------------
-template <typename T, int BM, int BN, int WM, int WN, bool GLDS>
+template <typename T, int BM, int BN, int WM, int WN, bool GLDS, bool F32 = false>
 static void launch_gemm_cfg(const GemmArgs& a, hipStream_t st) {
     constexpr int smem = 2 * (BM + BN) * GEMM_ROWB;
-    auto kern = gemm_mfma_kernel<T, BM, BN, WM, WN, GLDS>;
+    auto kern = gemm_mfma_kernel<T, BM, BN, WM, WN, GLDS, F32>;
     static bool attr_set = false;
     if (!attr_set) {
         LMX_CHECK_HIP(hipFuncSetAttribute(reinterpret_cast<const void*>(kern), hipFuncAttributeMaxDynamicSharedMemorySize, smem));
@@ -666,6 +668,7 @@ static void launch_gemm16(const GemmArgs& a, int variant, hipStream_t st) {
     // variant: 0 = auto, 2 = 128x128 reg-staged (kept as an independent cross-check of the LDS-DMA path), 4 = 64x128 glds, 5 = 64x64 glds,
     //          7 / 9 = LDS-ring kernels with counted vmcnt (128x256x64 3-slot, 256x256x64 2-slot; 8 waves), 15 = 64x64 4-slot ring (4 waves),
     //          18 = 128x128x64 2-slot 4 waves.  (Round 5 removed the arms auto never picks: 1, 12, 14 and the deeper rings 23 - 26 of round 4, EXPERIMENTS.md r4-C.)
+    if (a.c_f32) { launch_gemm_cfg<T, 64, 128, 2, 2, true, true>(a, st); return; }      // fp32 logits of a few wanted rows: one tile form
     if (variant == 0) {
         // Large problems: the ping-pong 256x256x64 kernel (gemm8p.hip), K-sliced when N = hidden leaves CUs idle and the caller brought
         // the partial-tile scratch (the engine does, per sequence; LMX_GEMM8P=0 switches the kernel off: the ring kernels below as an A/B and cross-check).
@@ -738,6 +741,7 @@ void launch_gemm(int dtype, const GemmArgs& a, int variant, hipStream_t st) {
         return;
     }
     LMX_REQUIRE(a.N % 8 == 0, "gemm: N must be a multiple of 8");
+    LMX_REQUIRE(!a.c_f32 || (!a.skw && !a.pk_kc && !a.qf_kc && !a.R && a.act != kActSiluMul), "gemm: fp32 output is for plain un-split linears");
     if (a.act == kActSiluMul) LMX_REQUIRE(a.N % 64 == 0, "gemm: SiLU·mul needs N (fused gate|up rows) % 64 == 0");
     if (dtype == kF32) {
         LMX_REQUIRE(a.K % 16 == 0, "gemm f32: K must be a multiple of 16");

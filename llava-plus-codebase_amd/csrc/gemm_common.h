@@ -73,7 +73,8 @@ __device__ __forceinline__ int lds_chunk_off(int row, int chunk) {
 // shared epilogue: acc[i][j][4q+e] = C[m = m_base + j*32 + l31][n = n_base + i*32 + 8q + 4hi + e]
 // (weight fragment = MFMA A operand, so a lane owns 4 consecutive n of one row m per accumulator quad)
 // ---------------------------------------------------------------------------------------------
-template <typename T, int MT, int NTL>
+// F32: the instantiation whose output is fp32 with an optional soft cap (GemmArgs::c_f32); its own template so that the hot kernels do not carry the branch
+template <typename T, int MT, int NTL, bool F32 = false>
 __device__ __forceinline__ void gemm_epilogue(const GemmArgs& a, f32x16 (&acc)[NTL][MT], int m_base, int n_base, int l31, int hi) {
     T* __restrict__ C = reinterpret_cast<T*>(a.C);
     const T* __restrict__ bias = reinterpret_cast<const T*>(a.bias);
@@ -177,7 +178,11 @@ __device__ __forceinline__ void gemm_epilogue(const GemmArgs& a, f32x16 (&acc)[N
 #pragma unroll
                     for (int e = 0; e < 4; ++e) v[e] += r[e];
                 }
-                store4<T>(C + (size_t)m * a.ldc + n, v);
+                if constexpr (F32) {
+#pragma unroll
+                    for (int e = 0; e < 4; ++e) v[e] = soft_cap(v[e], a.cap);
+                    store4<float>(reinterpret_cast<float*>(a.C) + (size_t)m * a.ldc + n, v);
+                } else store4<T>(C + (size_t)m * a.ldc + n, v);
             }
         }
     }

@@ -182,7 +182,8 @@ __device__ __forceinline__ void gemv2_body(const GemvArgs& a, int bid, char* sme
             const T tv = from_f32<T>(v);
             __hip_atomic_store(gran + n, ((unsigned long long)tag << 32) | (unsigned long long)tv.x, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
             if (ts && (bid & 31) == 31 && r == 0) __hip_atomic_fetch_max(ts + 7, (unsigned long long)__builtin_amdgcn_s_memrealtime(), __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
-        } else C[n] = from_f32<T>(v);
+        } else if (a.c_f32) reinterpret_cast<float*>(a.C)[n] = soft_cap(v, a.cap);
+        else C[n] = from_f32<T>(v);
     }
 }
 

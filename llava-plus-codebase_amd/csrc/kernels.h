@@ -34,6 +34,8 @@ struct GemmArgs {
     // belongs to image m / pk_rows at position m % pk_rows; per-image cache stride pk_img_stride elements.  pk_kc != null switches it on (any 16-bit GEMM
     // kernel that ends in gemm_epilogue; not SiLU*mul).
     void* pk_kc = nullptr; void* pk_vt = nullptr; int pk_heads = 0, pk_D = 0, pk_rows = 0, pk_spad = 0; size_t pk_img_stride = 0;
+    // fp32 output (an lm_head whose logits stay in 32 bits): C is float [M, ldc], every value passes soft_cap(v, cap) (cap = 0: none).  Un-split launches without residual.
+    int c_f32 = 0; float cap = 0.f;
 };
 void launch_gemm(int dtype, const GemmArgs& a, int variant, hipStream_t st);
 // true when launch_gemm(variant 0) of a [M, (nh + 2 nkv) D] x K projection runs as ONE un-split ping-pong launch whose tiles are head-aligned, i.e. can take
@@ -64,6 +66,7 @@ struct GemvArgs {
     int N, K;
     int ldx, ldw, ldc, ldr;
     int act;
+    int c_f32 = 0; float cap = 0.f;   // fp32 output with an optional soft cap, as GemmArgs::c_f32 (no SiLU*mul)
 };
 void launch_gemv(int dtype, const GemvArgs& a, int MB, hipStream_t st);
 // does launch_gemv(MB = 1) of this shape take the hand-counted weight stream (gemv2.h)?
@@ -85,6 +88,10 @@ struct FlashArgs {
     int causal;
     float* lse = nullptr;   // optional [n_heads][lse_stride]: log2-domain log-sum-exp of the scaled scores of every query row (the training backward's statistics)
     int lse_stride = 0;
+    // windowed form (causal only): row i sees keys j with 0 <= pos_i - j < window (0 = every earlier key); sink: a key of score 0 without a value joins the softmax;
+    // gate: head h's output row is multiplied by sigmoid(gate[row][h]) (model dtype, row pitch q_stride; null = off).  `win` switches the form on.
+    int win = 0, window = 0, sink = 0;
+    const void* gate = nullptr;
 };
 void launch_flash_prefill(int dtype, int D, const FlashArgs& a, hipStream_t st);
 
@@ -146,6 +153,43 @@ struct DecodeFusedArgs {
 void launch_decode_fused(int dtype, int D, const DecodeFusedArgs& a, hipStream_t st);
 size_t decode_fused_ws_floats(int n_heads, int n_split, int D);
 size_t decode_attn_ws_floats(int n_rows, int n_heads, int n_split, int D);
+
+// ---- layer-stack decoders (stack_ops.hip) ------------------------------------------------------------------------------------------------------------------
+// x_out = x_in + mult * rms_norm(y) * post_w + inject;  xn = rms_norm(x_out) * pre_w.  Any of x_in (= 0), y, inject, x_out, pre_w may be null.  The residual stream is
+// fp32 whatever the model dtype; rows have pitch H (a multiple of 8, zero padded), the norms' means run over H_real.  x_out may be x_in.
+struct ResidualNormArgs {
+    const float* x_in; const void* y; const void* post_w; const void* inject; const void* pre_w;
+    float* x_out; void* xn;
+    int H, H_real;
+    float mult, eps;
+};
+void launch_residual_norm(int dtype, const ResidualNormArgs& a, int rows, hipStream_t st);
+
+// rows of a prompt portion: q | k | v (| more) with head pitch D; per-head RMS norm over qk_dim (weights null = none), rotation of the first rot_dims dimensions (pairs
+// i, i + rot_dims / 2; table row = cos[rot_dims / 2] | sin[rot_dims / 2]), q back in place, k and v into the caches of launch_flash_prefill's layout
+struct QkvNormRopeArgs {
+    void* qkv; void* K; void* VT;
+    const void* q_norm; const void* k_norm;
+    const float* cos_sin;
+    int T, pos0, qkv_stride, n_heads, n_kv_heads, s_max, qk_dim, rot_dims;
+    float eps;
+};
+void launch_qkv_norm_rope_kv(int dtype, int D, const QkvNormRopeArgs& a, hipStream_t st);
+// attention of prompt rows on the vector ALUs (any dtype; FlashArgs' windowed causal form)
+void launch_rows_attn(int dtype, int D, const FlashArgs& a, hipStream_t st);
+
+// one new token per sequence: norm, rotation, append, windowed attention with sink and gate, one launch
+struct WinDecodeArgs {
+    const void* qkv; void* out;           // [n_seq][qkv_stride] rows q | k | v | gates; [n_seq][out_stride]
+    const void* q_norm; const void* k_norm; const float* cos_sin;
+    const DecodeFusedSeq* tab = nullptr;  // per sequence: caches of this layer, position, partials ([n_heads][n_split][D + 4] floats), tickets; null: `one`
+    DecodeFusedSeq one{};
+    int pos = -1;                         // position by value (one sequence whose length the host mirrors); < 0: read through pos_ptr
+    int n_seq = 1, qkv_stride = 0, out_stride = 0, n_heads = 0, n_kv_heads = 0, s_max = 0, n_split = 1;
+    int qk_dim = 0, rot_dims = 0, window = 0, sink = 0, gate_off = -1;      // gate_off: column of head 0's gate in the row, -1 = no gates
+    float scale = 1.f, eps = 0.f;
+};
+void launch_decode_win(int dtype, int D, const WinDecodeArgs& a, hipStream_t st);
 
 // ---- decode-step attention of a single request (decode_attn.hip; 16-bit models) ---------------------------------------------------------------------
 // RoPE(q, k_new) + KV append + attention over 128-key chunks + in-launch merge, position BY VALUE (the engine mirrors *d_len on the host), only the live
@@ -256,7 +300,7 @@ void launch_gather_tokens_batch(int dtype, const SeqStateRef* tab, int n, const 
 // then (embed != null) h_out[i] = embed[tok]: the next step's input row.  State comes from the device table `tab` (n members)
 // or from `single` (host pointer, passed by value; n must be 1).
 void launch_argmax_advance_batch(int dtype, const void* logits, int V, int ld, const SeqStateRef* tab, const SeqStateRef* single, int n, int64_t* ids_out,
-                                 const void* embed, void* h_out, int H, hipStream_t st);
+                                 const void* embed, void* h_out, int H, hipStream_t st, bool f32_logits = false);
 
 // ---- one-shot peer-to-peer all-reduce for decode-sized messages (p2p.hip) ---------------------------------------------
 constexpr int P2P_MAX_ROWS = 32;     // rows ([H] each) per launch = largest decode batch that goes through the skinny path

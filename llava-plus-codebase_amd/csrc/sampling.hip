@@ -332,10 +332,11 @@ void launch_sample(int dtype, const void* logits, int V, const SampleParams& p, 
 // End of a decode step, one workgroup per sequence: pick the next token (greedy argmax or a draw), advance the sequence state
 // (*len += 1, token log) and fetch the picked token's embedding row into the residual-stream row of the NEXT step — one launch
 // instead of argmax + advance + embedding gather.  `tab` (decode batch) or `single` (one sequence, by value) describes the state.
-template <typename T, int CPT>
+// T = logits, E = embedding rows (a model whose logits stay in 32 bits picks from float logits and fetches a 16-bit row)
+template <typename T, int CPT, typename E>
 __global__ __launch_bounds__(CPT > 0 ? FAST_NT : 1024) void pick_advance_batch_kernel(const T* __restrict__ logits_all, int V, int ld, const SeqStateRef* __restrict__ tab,
                                                                   SeqStateRef single, int64_t* __restrict__ ids_out,
-                                                                  const T* __restrict__ embed, T* __restrict__ h_out, int H) {
+                                                                  const E* __restrict__ embed, E* __restrict__ h_out, int H) {
     __shared__ SampleShared sh;
     __shared__ float bv[16];
     __shared__ int bi[16];
@@ -391,18 +392,20 @@ __global__ __launch_bounds__(CPT > 0 ? FAST_NT : 1024) void pick_advance_batch_k
         int64_t tt = t < 0 ? 0 : (t >= V ? V - 1 : t);
         const uint4* src = reinterpret_cast<const uint4*>(embed + (size_t)tt * H);
         uint4* dst = reinterpret_cast<uint4*>(h_out + (size_t)blockIdx.x * H);
-        for (int c = threadIdx.x; c < H * (int)sizeof(T) / 16; c += NT) dst[c] = src[c];
+        for (int c = threadIdx.x; c < H * (int)sizeof(E) / 16; c += NT) dst[c] = src[c];
     }
 }
 
 void launch_argmax_advance_batch(int dtype, const void* logits, int V, int ld, const SeqStateRef* tab, const SeqStateRef* single, int n, int64_t* ids_out,
-                                 const void* embed, void* h_out, int H, hipStream_t st) {
+                                 const void* embed, void* h_out, int H, hipStream_t st, bool f32_logits) {
     LMX_REQUIRE((tab != nullptr) != (single != nullptr) && (tab || n == 1), "pick: give a device table or one by-value state");
     const SeqStateRef one = single ? *single : SeqStateRef{};
-#define L2(TT, CC) hipLaunchKernelGGL((pick_advance_batch_kernel<TT, CC>), dim3(n), dim3(CC > 0 ? FAST_NT : 1024), 0, st, (const TT*)logits, V, ld, tab, one, \
-                                      ids_out, (const TT*)embed, (TT*)h_out, H)
-#define L(TT) do { if (sample_cpt(V) == 32) L2(TT, 32); else L2(TT, 0); } while (0)
-    if (dtype == kBF16) L(bf16_t); else if (dtype == kF16) L(f16_t); else L(float);
+#define L2(TT, CC, EE) hipLaunchKernelGGL((pick_advance_batch_kernel<TT, CC, EE>), dim3(n), dim3(CC > 0 ? FAST_NT : 1024), 0, st, (const TT*)logits, V, ld, tab, one, \
+                                          ids_out, (const EE*)embed, (EE*)h_out, H)
+#define L(TT, EE) do { if (sample_cpt(V) == 32) L2(TT, 32, EE); else L2(TT, 0, EE); } while (0)
+    if (dtype == kF32) L(float, float);
+    else if (dtype == kBF16) { if (f32_logits) L(float, bf16_t); else L(bf16_t, bf16_t); }
+    else { if (f32_logits) L(float, f16_t); else L(f16_t, f16_t); }
 #undef L
 #undef L2
     LMX_CHECK_HIP(hipGetLastError());

@@ -287,7 +287,8 @@ __global__ __launch_bounds__(NW * 64) void skinny_gemm_kernel(GemmArgs a) {
         if (bias) v += to_f32(bias[n]);
         if (a.act == kActQuickGelu) v = act_quick_gelu(v); else if (a.act == kActGeluErf) v = act_gelu_erf(v);
         if (Rr) v += to_f32(Rr[(size_t)m * a.ldr + n]);
-        C[(size_t)m * a.ldc + n] = from_f32<T>(v);
+        if (a.c_f32) reinterpret_cast<float*>(a.C)[(size_t)m * a.ldc + n] = soft_cap(v, a.cap);
+        else C[(size_t)m * a.ldc + n] = from_f32<T>(v);
     }
 }
 

@@ -1,0 +1,465 @@
+// Layer-stack decoders: a model described layer by layer (include/llava_mi355x.h: lmx_stack_config / lmx_layer_config) on the engine's own sequences, caches, decode
+// batches, samplers and linears.  What differs from the LLaMA decoder of engine.cpp:
+//
+//   * the residual stream is fp32 in every model dtype; a sublayer's output is normalised before it is added (times residual_mult), so no linear adds a residual in its
+//     epilogue — residual_norm (stack_ops.hip) does post-norm, addition and the next sublayer's pre-norm in one launch between any two linears;
+//   * a range of layers may run several times in a row (loop): weights exist once per LAYER, caches once per layer RUN; before each pass but the first the embedding row
+//     is added to the residual (inject), in the launch that ends the previous layer;
+//   * per layer: head counts and widths, query / key norm, partial rotation, score scale, window, softmax sink, output gates, feed-forward width (or none);
+//   * logits are fp32 and soft-capped in the lm_head's epilogue.
+//
+// Layout: width and ff are padded to multiples of 64, head vectors to D in {64, 128, 256}, the vocabulary to 8, all with zero weights, so that padded lanes stay zero
+// through every op (norm means divide by the true sizes).  One fused q | k | v | gate weight per layer; gate | up interleaved as in the LLaMA decoder.
+#include "engine.h"
+
+#include <cstring>
+
+namespace lmx {
+
+static int round_up(int a, int b) { return (a + b - 1) / b * b; }
+
+Model::Model(const lmx_stack_config& c, const lmx_layer_config* layers) {
+    LMX_REQUIRE(c.abi_version == LMX_ABI_VERSION, "lmx_stack_config.abi_version mismatch");
+    LMX_REQUIRE(c.dtype == kF32 || c.dtype == kBF16 || c.dtype == kF16, "bad dtype");
+    LMX_REQUIRE(c.width >= 1 && c.vocab_size >= 1 && c.n_layers >= 1 && layers, "stack: empty model");
+    LMX_REQUIRE(c.loop_times >= 1 && c.loop_start >= 0 && c.loop_start <= c.loop_stop && c.loop_stop <= c.n_layers, "stack: bad loop range");
+    cfg.abi_version = c.abi_version; cfg.dtype = c.dtype; cfg.hidden_size = c.width; cfg.vocab_size = c.vocab_size; cfg.n_layers = c.n_layers;
+    cfg.rms_eps = c.norm_eps; cfg.max_position = c.max_position; cfg.tp_world = 1; cfg.tp_rank = 0; cfg.gemm_variant = c.gemm_variant;
+    es = (int)dtype_size(c.dtype);
+    stk = std::make_unique<Stack>();
+    Stack& S = *stk;
+    S.c = c;
+    H = round_up(c.width, 64);
+    LMX_REQUIRE(H <= 8192, "stack: width up to 8192");
+    V = round_up(c.vocab_size, 8); Vr = c.vocab_size; V_l = V; v_off = 0;
+    les = 4;
+    s_max = round_up(c.max_position > 0 ? c.max_position : 2048, 128);
+    S.layers.resize((size_t)c.n_layers);
+    for (int i = 0; i < c.n_layers; ++i) {
+        StackLayer& l = S.layers[(size_t)i];
+        const lmx_layer_config& d = l.c = layers[i];
+        LMX_REQUIRE(d.n_heads >= 1 && d.n_kv_heads >= 1 && d.n_heads % d.n_kv_heads == 0, "stack: n_heads must be a multiple of n_kv_heads");
+        LMX_REQUIRE(d.qk_dim >= 1 && d.v_dim >= 1 && d.qk_dim <= 256 && d.v_dim <= 256, "stack: head widths up to 256");
+        LMX_REQUIRE(d.rope_dims >= 0 && d.rope_dims % 2 == 0 && d.rope_dims <= d.qk_dim, "stack: rotated dimensions must be even and inside the head");
+        LMX_REQUIRE(d.rope_dims == 0 || (d.rope_table >= 0 && d.rope_table < 256), "stack: bad rope table index");
+        LMX_REQUIRE(d.window >= 0 && d.ff >= 0, "stack: bad window / feed-forward width");
+        const int m = std::max(d.qk_dim, d.v_dim);
+        l.D = m <= 64 ? 64 : m <= 128 ? 128 : 256;
+        l.gate_off = d.out_gate ? (d.n_heads + 2 * d.n_kv_heads) * l.D : -1;
+        l.qkv_n = (d.n_heads + 2 * d.n_kv_heads) * l.D + (d.out_gate ? round_up(d.n_heads, 64) : 0);
+        l.ff = round_up(d.ff, 64);
+        if (d.rope_dims && d.rope_table >= (int)S.rope.size()) { S.rope.resize((size_t)d.rope_table + 1, nullptr); S.rope_dims.resize((size_t)d.rope_table + 1, 0); }
+        // sizes the shared workspaces (Seq, Batch) are cut by: the widest layer
+        D = std::max(D, l.D); nh_l = std::max(nh_l, d.n_heads); nkv_l = std::max(nkv_l, d.n_kv_heads);
+        qkv_n = std::max(qkv_n, l.qkv_n); I_l = std::max(I_l, std::max(l.ff, 64)); S.attn_n = std::max(S.attn_n, d.n_heads * l.D);
+        S.dec_ws = std::max(S.dec_ws, decode_fused_ws_floats(d.n_heads, std::min((s_max + 127) / 128, 32), l.D));
+    }
+    auto run = [&](int layer, bool inject) {
+        const StackLayer& l = S.layers[(size_t)layer];
+        const size_t bytes = ((size_t)l.c.n_kv_heads * s_max * l.D * es + 255) / 256 * 256;
+        S.runs.push_back(StackRun{layer, inject, S.kv_bytes});
+        S.kv_bytes += bytes;
+    };
+    for (int i = 0; i < c.loop_start; ++i) run(i, false);
+    for (int t = 0; t < c.loop_times; ++t)
+        for (int i = c.loop_start; i < c.loop_stop; ++i) run(i, t > 0 && i == c.loop_start);
+    for (int i = c.loop_stop; i < c.n_layers; ++i) run(i, false);
+    L = (int)S.runs.size();
+    LMX_REQUIRE(L >= 1, "stack: no layer runs");
+    LMX_CHECK_HIP(hipEventCreateWithFlags(&vws_done, hipEventDisableTiming));
+}
+
+void Model::stack_set_rope(int table, int dims, const float* host, int n_pos) {
+    LMX_REQUIRE(stk, "not a layer-stack model");
+    LMX_REQUIRE(table >= 0 && table < (int)stk->rope.size() && dims > 0 && host && n_pos >= s_max, "rope table: bad index or too few positions");
+    float*& p = stk->rope[(size_t)table];
+    if (p) { (void)hipFree(p); p = nullptr; }
+    LMX_CHECK_HIP(hipMalloc(reinterpret_cast<void**>(&p), (size_t)n_pos * dims * sizeof(float)));
+    LMX_CHECK_HIP(hipMemcpy(p, host, (size_t)n_pos * dims * sizeof(float), hipMemcpyHostToDevice));
+    stk->rope_dims[(size_t)table] = dims;
+}
+
+// ---------------------------------------------------------------------------------------------------------------
+// weights.  Names: embed, head, final.norm, and per layer l<i>.{norm1, norm1b, norm2, norm2b, mix.{q, k, v}[.b], mix.{q, k}.norm, mix.g, mix.o, mlp.{gate, up, down}}
+// ---------------------------------------------------------------------------------------------------------------
+void Model::stack_load_weight(const std::string& name, const void* src, int ndim, const int64_t* shape, hipStream_t st) {
+    Stack& S = *stk;
+    const int W = S.c.width, dt = cfg.dtype;
+    auto expect = [&](std::initializer_list<int64_t> want) {
+        bool ok = (int)want.size() == ndim;
+        int i = 0;
+        for (auto w : want) { if (ok && shape[i] != w) ok = false; ++i; }
+        if (ok) return;
+        std::string got = "[", exp = "[";
+        for (int k = 0; k < ndim; ++k) got += std::to_string(shape[k]) + ",";
+        for (auto w : want) exp += std::to_string(w) + ",";
+        throw Error{"shape mismatch for " + name + ": got " + got + "] expected " + exp + "]"};
+    };
+    // rows [0, rows) x cols of a [rows][cols] source into dst (pitch dst_cols) at (row0, col0)
+    auto block = [&](void* dst, int dst_cols, int row0, int col0, const void* s, int src_cols, int rows, int cols) {
+        LMX_CHECK_HIP(hipMemcpy2DAsync(static_cast<char*>(dst) + ((size_t)row0 * dst_cols + col0) * es, (size_t)dst_cols * es, s, (size_t)src_cols * es, (size_t)cols * es,
+                                       (size_t)rows, hipMemcpyDeviceToDevice, st));
+    };
+    auto at = [&](size_t elems) { return static_cast<const char*>(src) + elems * es; };
+    auto vec = [&](void*& dst, int n, int padded) {
+        expect({n});
+        if (!dst) dst = alloc_weight((size_t)padded * es, true);
+        block(dst, padded, 0, 0, src, n, 1, n);
+    };
+    auto table = [&](void*& dst) {
+        expect({S.c.vocab_size, W});
+        if (!dst) dst = alloc_weight((size_t)V * H * es, true);
+        block(dst, H, 0, 0, src, W, S.c.vocab_size, W);
+    };
+    if (name == "embed") table(embed);
+    else if (name == "head") table(lm_head);
+    else if (name == "final.norm") vec(final_norm, W, H);
+    else {
+        const size_t dot = name.find('.');
+        LMX_REQUIRE(name.size() > 2 && name[0] == 'l' && dot != std::string::npos && dot > 1, "unknown tensor name: " + name);
+        for (size_t k = 1; k < dot; ++k) LMX_REQUIRE(name[k] >= '0' && name[k] <= '9', "unknown tensor name: " + name);
+        const int li = atoi(name.substr(1, dot - 1).c_str());
+        LMX_REQUIRE(li >= 0 && li < S.c.n_layers, "layer index out of range: " + name);
+        const std::string sub = name.substr(dot + 1);
+        StackLayer& l = S.layers[(size_t)li];
+        const lmx_layer_config& d = l.c;
+        if (!l.wqkv) {
+            l.wqkv = alloc_weight((size_t)l.qkv_n * H * es, true);
+            if (d.qkv_bias) l.bqkv = alloc_weight((size_t)l.qkv_n * es, true);
+            l.wo = alloc_weight((size_t)H * d.n_heads * l.D * es, true);
+            if (l.ff) { l.wgu = alloc_weight((size_t)2 * l.ff * H * es, true); l.wd = alloc_weight((size_t)H * l.ff * es, true); }
+        }
+        auto heads = [&](int first_slot, int n, int dim) {                    // [n * dim][W] -> one padded head block per head
+            expect({(int64_t)n * dim, W});
+            for (int h = 0; h < n; ++h) block(l.wqkv, H, (first_slot + h) * l.D, 0, at((size_t)h * dim * W), W, dim, W);
+        };
+        auto head_bias = [&](int first_slot, int n, int dim) {
+            LMX_REQUIRE(d.qkv_bias, "projection bias given but the layer has none: " + name);
+            expect({(int64_t)n * dim});
+            block(l.bqkv, l.D, first_slot, 0, src, dim, n, dim);
+        };
+        auto gate_up = [&](int half) {
+            LMX_REQUIRE(d.ff > 0, "feed-forward tensor given but the layer has none: " + name);
+            expect({d.ff, W});
+            DevBuf tmp;                                                       // rows padded to whole 32-row groups and columns to the padded width
+            tmp.ensure((size_t)l.ff * H * es, true);
+            block(tmp.p, H, 0, 0, src, W, d.ff, W);
+            launch_interleave_half(dt, tmp.p, l.wgu, l.ff, H, half, st);
+            LMX_CHECK_HIP(hipStreamSynchronize(st));
+        };
+        const int nh = d.n_heads, nk = d.n_kv_heads;
+        if (sub == "norm1") vec(l.n1, W, H);
+        else if (sub == "norm1b") vec(l.n1b, W, H);
+        else if (sub == "norm2" && d.ff) vec(l.n2, W, H);
+        else if (sub == "norm2b" && d.ff) vec(l.n2b, W, H);
+        else if (sub == "mix.q") heads(0, nh, d.qk_dim);
+        else if (sub == "mix.k") heads(nh, nk, d.qk_dim);
+        else if (sub == "mix.v") heads(nh + nk, nk, d.v_dim);
+        else if (sub == "mix.q.b") head_bias(0, nh, d.qk_dim);
+        else if (sub == "mix.k.b") head_bias(nh, nk, d.qk_dim);
+        else if (sub == "mix.v.b") head_bias(nh + nk, nk, d.v_dim);
+        else if (sub == "mix.q.norm" && d.qk_norm) vec(l.qn, d.qk_dim, l.D);
+        else if (sub == "mix.k.norm" && d.qk_norm) vec(l.kn, d.qk_dim, l.D);
+        else if (sub == "mix.g" && d.out_gate) { expect({nh, W}); block(l.wqkv, H, l.gate_off, 0, src, W, nh, W); }
+        else if (sub == "mix.o") {
+            expect({W, (int64_t)nh * d.v_dim});
+            for (int h = 0; h < nh; ++h) block(l.wo, nh * l.D, 0, h * l.D, at((size_t)h * d.v_dim), nh * d.v_dim, W, d.v_dim);
+        }
+        else if (sub == "mlp.gate") gate_up(0);
+        else if (sub == "mlp.up") gate_up(1);
+        else if (sub == "mlp.down" && d.ff) { expect({W, d.ff}); block(l.wd, l.ff, 0, 0, src, d.ff, W, d.ff); }
+        else throw Error{"unknown tensor name: " + name};
+    }
+    loaded.insert(name);
+}
+
+void Model::stack_finalize() {
+    std::string missing;
+    auto need = [&](const std::string& n) { if (!loaded.count(n)) missing += n + " "; };
+    need("embed"); need("head"); need("final.norm");
+    for (int i = 0; i < stk->c.n_layers; ++i) {
+        const lmx_layer_config& d = stk->layers[(size_t)i].c;
+        const std::string p = "l" + std::to_string(i) + ".";
+        for (const char* s : {"norm1", "norm1b", "mix.q", "mix.k", "mix.v", "mix.o"}) need(p + s);
+        if (d.qkv_bias) for (const char* s : {"mix.q.b", "mix.k.b", "mix.v.b"}) need(p + s);
+        if (d.qk_norm) for (const char* s : {"mix.q.norm", "mix.k.norm"}) need(p + s);
+        if (d.out_gate) need(p + "mix.g");
+        if (d.ff) for (const char* s : {"norm2", "norm2b", "mlp.gate", "mlp.up", "mlp.down"}) need(p + s);
+        if (d.rope_dims) {
+            const bool ok = stk->rope[(size_t)d.rope_table] && stk->rope_dims[(size_t)d.rope_table] == d.rope_dims;
+            if (!ok) missing += "<rope table " + std::to_string(d.rope_table) + "> ";
+        }
+    }
+    if (!missing.empty()) throw Error{"missing tensors: " + missing};
+}
+
+void Model::stack_batch_weights(hipStream_t st) {
+    auto mk = [&](const void* W, int N, int K) -> void* {
+        if (!W) return nullptr;
+        void* d = alloc_weight(skinny_swizzled_bytes(N, K, es));
+        launch_skinny_swizzle(cfg.dtype, W, K, d, N, K, st);
+        return d;
+    };
+    for (StackLayer& l : stk->layers) {
+        l.sw_qkv = mk(l.wqkv, l.qkv_n, H);
+        l.sw_o = mk(l.wo, H, l.c.n_heads * l.D);
+        l.sw_gu = mk(l.wgu, 2 * l.ff, H);
+        l.sw_d = mk(l.wd, H, l.ff);
+    }
+    sw_lm_head = mk(lm_head, V, H);
+    LMX_CHECK_HIP(hipStreamSynchronize(st));
+}
+
+// what ends sublayer `sub` (0 mixer, 1 feed-forward) of run r: its post-norm, the injected rows if the next run wants them, and the norm in front of the next linear
+struct StackStep { const void* post; const void* pre; bool inject; };
+static StackStep stack_step(const Stack& S, int r, int sub, const void* final_norm) {
+    const StackLayer& l = S.layers[(size_t)S.runs[(size_t)r].layer];
+    if (sub == 0 && l.ff) return {l.n1b, l.n2, false};
+    const void* post = sub == 0 ? l.n1b : l.n2b;
+    if (r + 1 == (int)S.runs.size()) return {post, final_norm, false};
+    const StackRun& nx = S.runs[(size_t)r + 1];
+    return {post, S.layers[(size_t)nx.layer].n1, nx.inject};
+}
+
+static QkvNormRopeArgs rope_args(const Stack& S, const StackLayer& l, void* qkv, void* kc, void* vt, int T, int pos0, int s_max) {
+    const lmx_layer_config& d = l.c;
+    return QkvNormRopeArgs{qkv, kc, vt, l.qn, l.kn, d.rope_dims ? S.rope[(size_t)d.rope_table] : nullptr, T, pos0, l.qkv_n, d.n_heads, d.n_kv_heads, s_max, d.qk_dim, d.rope_dims, S.c.norm_eps};
+}
+
+// ---------------------------------------------------------------------------------------------------------------
+// prefill: one sequence or several packed, as Model::prefill_multi walks them (pieces of block_rows rows; linears over the piece, attention per segment)
+// ---------------------------------------------------------------------------------------------------------------
+void Model::stack_prefill(Seq* const* seqs, const void* const* embeds, const int* Ts, int n, int block_rows, bool greedy, const StackOutputs& out, hipStream_t st) {
+    Stack& S = *stk;
+    LMX_REQUIRE(n >= 1 && seqs && embeds && Ts, "prefill: bad arguments");
+    long total = 0;
+    for (int i = 0; i < n; ++i) {
+        LMX_REQUIRE(seqs[i] && seqs[i]->m == this && embeds[i] && Ts[i] > 0, "prefill: bad sequence / input");
+        LMX_REQUIRE(seqs[i]->len + Ts[i] <= s_max, "prefill: sequence would exceed the KV-cache capacity (max_position)");
+        for (int j = 0; j < i; ++j) LMX_REQUIRE(seqs[j] != seqs[i], "prefill: the same sequence appears twice");
+        seqs[i]->last_stream = st; seqs[i]->used = true;
+        total += Ts[i];
+    }
+    LMX_REQUIRE(!out.hidden || n == 1, "prefill: the residual trace is for one sequence");
+    if (block_rows <= 0 || block_rows > total) block_rows = (int)total;
+    const int dt = cfg.dtype, gv = cfg.gemm_variant;
+    Seq* s0 = seqs[0];
+    constexpr int LOGIT_ROWS = 1024;                     // rows of one lm_head launch
+    size_t off = 0;
+    auto carve = [&](size_t bytes) { size_t o = off; off += (bytes + 255) / 256 * 256; return o; };
+    const size_t o_h = carve((size_t)block_rows * H * es), o_xr = carve((size_t)block_rows * H * 4), o_x = carve((size_t)block_rows * H * es),
+                 o_y = carve((size_t)block_rows * H * es), o_qkv = carve((size_t)block_rows * qkv_n * es), o_attn = carve((size_t)block_rows * S.attn_n * es),
+                 o_act = carve((size_t)block_rows * I_l * es), o_log = carve((size_t)V * 4), o_want = carve((size_t)std::min(block_rows, LOGIT_ROWS) * H * es);
+    if (off > s0->pws.bytes) { LMX_CHECK_HIP(hipStreamSynchronize(st)); s0->pws.ensure(off); }
+    char* Wk = s0->pws.as<char>();
+    void *h = Wk + o_h, *x = Wk + o_x, *y = Wk + o_y, *qkv = Wk + o_qkv, *attn = Wk + o_attn, *act = Wk + o_act, *want = Wk + o_want;
+    float *xr = reinterpret_cast<float*>(Wk + o_xr), *last_logits = reinterpret_cast<float*>(Wk + o_log);
+    if (dt != kF32 && !s0->skw.p) {
+        LMX_CHECK_HIP(hipStreamSynchronize(st));
+        s0->skw.ensure((size_t)256 * 256 * 256 * sizeof(float));
+    }
+    auto with_scratch = [&](GemmArgs g) { g.skw = s0->skw.p; return g; };
+    auto rows = [&](void* base, long r0, size_t width) { return static_cast<char*>(base) + (size_t)r0 * width * es; };
+    auto norm = [&](const float* xi, const void* yy, const StackStep& sp, int nr, bool with_inject = true, bool with_pre = true) {
+        LMX_PROF("prefill.residual_norm");
+        launch_residual_norm(dt, ResidualNormArgs{xi, yy, sp.post, with_inject && sp.inject ? h : nullptr, with_pre ? sp.pre : nullptr, xr, x, H, S.c.width, S.c.residual_mult, S.c.norm_eps}, nr, st);
+    };
+    struct Segment { int seq, src0, dst0, n, pos0; };
+    int cur = 0, cur_done = 0;
+    std::vector<int> want_next((size_t)n, 0), want_base((size_t)n, 0);      // wanted rows already served / first output row of each sequence
+    for (int i = 1; i < n; ++i) want_base[(size_t)i] = want_base[(size_t)i - 1] + (out.logits ? (out.want ? (int)out.want[i - 1].size() : Ts[i - 1]) : 0);
+    while (cur < n) {
+        std::vector<Segment> seg;
+        int fill = 0;
+        while (cur < n && fill < block_rows) {
+            const int take = std::min(block_rows - fill, Ts[cur] - cur_done);
+            seg.push_back(Segment{cur, cur_done, fill, take, seqs[cur]->len + cur_done});
+            fill += take; cur_done += take;
+            if (cur_done == Ts[cur]) { ++cur; cur_done = 0; }
+        }
+        for (const Segment& g : seg)
+            LMX_CHECK_HIP(hipMemcpyAsync(rows(h, g.dst0, H), static_cast<const char*>(embeds[g.seq]) + (size_t)g.src0 * H * es, (size_t)g.n * H * es, hipMemcpyDeviceToDevice, st));
+        norm(nullptr, nullptr, StackStep{nullptr, S.layers[(size_t)S.runs[0].layer].n1, true}, fill);      // x = the embedding rows
+        for (int r = 0; r < L; ++r) {
+            const StackLayer& l = S.layers[(size_t)S.runs[(size_t)r].layer];
+            const lmx_layer_config& d = l.c;
+            const int an = d.n_heads * l.D;
+            { LMX_PROF_K("prefill.gemm.qkv"); launch_gemm(dt, with_scratch(GemmArgs{x, l.wqkv, qkv, l.bqkv, nullptr, fill, l.qkv_n, H, H, H, l.qkv_n, 0, kActNone}), gv, st); }
+            for (const Segment& g : seg) {
+                Seq* s = seqs[g.seq];
+                void *kc = s->kc.as<char>() + S.runs[(size_t)r].kv_off, *vt = s->vt.as<char>() + S.runs[(size_t)r].kv_off;
+                void *qr = rows(qkv, g.dst0, l.qkv_n), *ar = rows(attn, g.dst0, an);
+                { LMX_PROF("prefill.norm_rope_kv"); launch_qkv_norm_rope_kv(dt, l.D, rope_args(S, l, qr, kc, vt, g.n, g.pos0, s_max), st); }
+                LMX_PROF("prefill.attn");
+                FlashArgs fa{qr, ar, kc, vt, g.n, g.pos0 + g.n, g.pos0, l.qkv_n, an, d.n_heads, d.n_kv_heads, s_max, d.attn_scale, 1};
+                fa.win = 1; fa.window = d.window; fa.sink = d.softmax_sink; fa.gate = l.gate_off >= 0 ? static_cast<char*>(qr) + (size_t)l.gate_off * es : nullptr;
+                if (dt == kF32 || l.D > 128) launch_rows_attn(dt, l.D, fa, st); else launch_flash_prefill(dt, l.D, fa, st);
+            }
+            { LMX_PROF_K("prefill.gemm.o"); launch_gemm(dt, with_scratch(GemmArgs{attn, l.wo, y, nullptr, nullptr, fill, H, an, an, an, H, 0, kActNone}), gv, st); }
+            if (l.ff) {
+                norm(xr, y, stack_step(S, r, 0, final_norm), fill);
+                { LMX_PROF_K("prefill.gemm.gate_up"); launch_gemm(dt, with_scratch(GemmArgs{x, l.wgu, act, nullptr, nullptr, fill, 2 * l.ff, H, H, H, l.ff, 0, kActSiluMul}), gv, st); }
+                { LMX_PROF_K("prefill.gemm.down"); launch_gemm(dt, with_scratch(GemmArgs{act, l.wd, y, nullptr, nullptr, fill, H, l.ff, l.ff, l.ff, H, 0, kActNone}), gv, st); }
+            }
+            const StackStep sp = stack_step(S, r, l.ff ? 1 : 0, final_norm);
+            if (out.hidden) {
+                // residual trace: the stream right after this run, before anything the next run adds
+                norm(xr, y, sp, fill, false, false);
+                LMX_CHECK_HIP(hipMemcpyAsync(out.hidden + ((size_t)r * Ts[0] + seg[0].src0) * H, xr, (size_t)fill * H * 4, hipMemcpyDeviceToDevice, st));
+                norm(xr, nullptr, sp, fill);
+            } else norm(xr, y, sp, fill);
+        }
+        // logits of the wanted rows of this piece (x holds the finally normalised rows)
+        if (out.logits)
+            for (const Segment& g : seg) {
+                std::vector<int> rws;                     // rows of this segment, ascending (relative to the sequence's new rows)
+                if (!out.want) { rws.resize((size_t)g.n); for (int i = 0; i < g.n; ++i) rws[(size_t)i] = g.src0 + i; }
+                else { const auto& w = out.want[g.seq]; int& p = want_next[(size_t)g.seq]; while (p + (int)rws.size() < (int)w.size() && w[(size_t)p + rws.size()] < g.src0 + g.n) rws.push_back(w[(size_t)p + rws.size()]); }
+                for (size_t r0 = 0; r0 < rws.size(); r0 += LOGIT_ROWS) {
+                    const int nr = (int)std::min(rws.size() - r0, (size_t)std::min(block_rows, LOGIT_ROWS));
+                    for (int i = 0; i < nr;) {            // consecutive rows in one copy
+                        int k = i + 1;
+                        while (k < nr && rws[r0 + k] == rws[r0 + k - 1] + 1) ++k;
+                        LMX_CHECK_HIP(hipMemcpyAsync(rows(want, i, H), rows(x, g.dst0 + rws[r0 + i] - g.src0, H), (size_t)(k - i) * H * es, hipMemcpyDeviceToDevice, st));
+                        i = k;
+                    }
+                    GemmArgs ga{want, lm_head, out.logits + (size_t)(want_base[(size_t)g.seq] + want_next[(size_t)g.seq]) * V, nullptr, nullptr, nr, V, H, H, H, V, 0, kActNone};
+                    ga.c_f32 = 1; ga.cap = S.c.logit_softcap;
+                    { LMX_PROF("prefill.gemm.lm_head"); launch_gemm(dt, ga, gv, st); }
+                    want_next[(size_t)g.seq] += nr;
+                }
+            }
+        for (const Segment& g : seg) {
+            if (g.src0 + g.n != Ts[g.seq] || !(greedy || out.last_logits)) continue;
+            Seq* s = seqs[g.seq];
+            float* dst = out.last_logits ? out.last_logits + (size_t)g.seq * V : last_logits;
+            GemvArgs ga{rows(x, g.dst0 + g.n - 1, H), lm_head, dst, nullptr, nullptr, nullptr, 0.f, V, H, H, H, V, 0, kActNone};
+            ga.c_f32 = 1; ga.cap = S.c.logit_softcap;
+            { LMX_PROF_K("prefill.gemv.lm_head"); launch_gemv(dt, ga, 1, st); }
+            if (!greedy) continue;
+            if (s->samp.temperature > 0.f) launch_sample(kF32, dst, Vr, s->samp, s->d_nout, s->d_tok, nullptr, nullptr, st);
+            else launch_argmax(kF32, dst, Vr, s->d_tok, st);
+            launch_log_token(s->d_tok, s->d_log, s->d_nout, s->log_cap, s->d_stop, st);
+        }
+    }
+    for (int i = 0; i < n; ++i) {
+        seqs[i]->len += Ts[i];
+        launch_set_state(seqs[i]->d_len, seqs[i]->len, seqs[i]->d_tok, 0, 0, seqs[i]->d_nout, -1, st);
+    }
+}
+
+// ---------------------------------------------------------------------------------------------------------------
+// decode
+// ---------------------------------------------------------------------------------------------------------------
+static WinDecodeArgs decode_args(const Stack& S, const StackLayer& l, const void* qkv, void* out, int n_seq, int max_len, int s_max) {
+    const lmx_layer_config& d = l.c;
+    WinDecodeArgs a;
+    a.qkv = qkv; a.out = out; a.q_norm = l.qn; a.k_norm = l.kn; a.cos_sin = d.rope_dims ? S.rope[(size_t)d.rope_table] : nullptr;
+    a.n_seq = n_seq; a.qkv_stride = l.qkv_n; a.out_stride = d.n_heads * l.D; a.n_heads = d.n_heads; a.n_kv_heads = d.n_kv_heads; a.s_max = s_max;
+    a.qk_dim = d.qk_dim; a.rot_dims = d.rope_dims; a.window = d.window; a.sink = d.softmax_sink; a.gate_off = l.gate_off; a.scale = d.attn_scale; a.eps = S.c.norm_eps;
+    // chunks the longest member's window can touch; enough workgroups to fill the chip, no more
+    int span = max_len + 1;
+    if (d.window > 0 && d.window + 127 < span) span = d.window + 127;
+    const int chunks = std::max(1, std::min((span + 127) / 128, 32));
+    const int fill = (1024 + d.n_heads * n_seq - 1) / (d.n_heads * n_seq);
+    a.n_split = std::max(1, std::min(chunks, fill));
+    return a;
+}
+
+void Model::stack_decode_step(Seq* s, hipStream_t st, int64_t* id_out) {
+    Stack& S = *stk;
+    const int dt = cfg.dtype;
+    float* xr = s->d_xr;
+    auto norm = [&](const float* xi, const void* yy, const StackStep& sp) {
+        LMX_PROF_K("decode.residual_norm");
+        launch_residual_norm(dt, ResidualNormArgs{xi, yy, sp.post, sp.inject ? s->d_h : nullptr, sp.pre, xr, s->d_x, H, S.c.width, S.c.residual_mult, S.c.norm_eps}, 1, st);
+    };
+    auto gemv = [&](const char* name, const void* xin, const void* w, void* c, const void* bias, int N, int K, int act) {
+        LMX_PROF_K(name);
+        launch_gemv(dt, GemvArgs{xin, w, c, bias, nullptr, nullptr, 0.f, N, K, K, K, N, 0, act}, 1, st);
+    };
+    norm(nullptr, nullptr, StackStep{nullptr, S.layers[(size_t)S.runs[0].layer].n1, true});
+    for (int r = 0; r < L; ++r) {
+        const StackLayer& l = S.layers[(size_t)S.runs[(size_t)r].layer];
+        const int an = l.c.n_heads * l.D;
+        gemv("decode.gemv.qkv", s->d_x, l.wqkv, s->d_qkv, l.bqkv, l.qkv_n, H, kActNone);
+        {
+            LMX_PROF_K("decode.attn");
+            WinDecodeArgs a = decode_args(S, l, s->d_qkv, s->d_attn, 1, s->len, s_max);
+            a.one = DecodeFusedSeq{s->kc.as<char>() + S.runs[(size_t)r].kv_off, s->vt.as<char>() + S.runs[(size_t)r].kv_off, s->d_len, s->d_aws, s->d_cnt};
+            a.pos = s->len;
+            launch_decode_win(dt, l.D, a, st);
+        }
+        gemv("decode.gemv.o", s->d_attn, l.wo, s->d_y, nullptr, H, an, kActNone);
+        if (l.ff) {
+            norm(xr, s->d_y, stack_step(S, r, 0, final_norm));
+            gemv("decode.gemv.gate_up", s->d_x, l.wgu, s->d_act, nullptr, 2 * l.ff, H, kActSiluMul);
+            gemv("decode.gemv.down", s->d_act, l.wd, s->d_y, nullptr, H, l.ff, kActNone);
+        }
+        norm(xr, s->d_y, stack_step(S, r, l.ff ? 1 : 0, final_norm));
+    }
+    {
+        LMX_PROF_K("decode.gemv.lm_head");
+        GemvArgs ga{s->d_x, lm_head, s->d_logits, nullptr, nullptr, nullptr, 0.f, V, H, H, H, V, 0, kActNone};
+        ga.c_f32 = 1; ga.cap = S.c.logit_softcap;
+        launch_gemv(dt, ga, 1, st);
+    }
+    LMX_PROF("decode.argmax");
+    const SeqStateRef ref{s->d_len, s->d_nout, s->d_tok, s->d_log, s->log_cap, 0, s->samp, s->d_stop};
+    launch_argmax_advance_batch(dt, s->d_logits, Vr, V, nullptr, &ref, 1, id_out, embed, s->d_h, H, st, /*f32_logits=*/true);
+}
+
+void Model::stack_decode_batch_step(Batch* b, Seq* const* seqs, int n, int64_t* ids, hipStream_t st) {
+    Stack& S = *stk;
+    const int dt = cfg.dtype;
+    auto norm = [&](const float* xi, const void* yy, const StackStep& sp) {
+        LMX_PROF("decode_batch.residual_norm");
+        launch_residual_norm(dt, ResidualNormArgs{xi, yy, sp.post, sp.inject ? b->h : nullptr, sp.pre, b->xr, b->x, H, S.c.width, S.c.residual_mult, S.c.norm_eps}, n, st);
+    };
+    auto linear = [&](GemmArgs g, const void* wsw) {
+        LMX_PROF("decode_batch.linear");
+        if (dt != kF32 && n <= 32) {
+            g.Wsw = wsw;
+            if (!g.c_f32) { g.skw = b->sk_scratch.p; g.sk_cnt = b->sk_cnt.as<int>(); }
+            launch_skinny_gemm(dt, g, st);
+        } else launch_gemm(dt, g, cfg.gemm_variant, st);
+    };
+    int max_len = 0;
+    for (int i = 0; i < n; ++i) max_len = std::max(max_len, seqs[i]->len);
+    norm(nullptr, nullptr, StackStep{nullptr, S.layers[(size_t)S.runs[0].layer].n1, true});
+    for (int r = 0; r < L; ++r) {
+        const StackLayer& l = S.layers[(size_t)S.runs[(size_t)r].layer];
+        const int an = l.c.n_heads * l.D;
+        linear(GemmArgs{b->x, l.wqkv, b->qkv, l.bqkv, nullptr, n, l.qkv_n, H, H, H, l.qkv_n, 0, kActNone}, l.sw_qkv);
+        {
+            LMX_PROF("decode_batch.attn");
+            WinDecodeArgs a = decode_args(S, l, b->qkv, b->attn, n, max_len, s_max);
+            a.tab = b->d_attn_tab + (size_t)r * b->cap;
+            launch_decode_win(dt, l.D, a, st);
+        }
+        linear(GemmArgs{b->attn, l.wo, b->y, nullptr, nullptr, n, H, an, an, an, H, 0, kActNone}, l.sw_o);
+        if (l.ff) {
+            norm(b->xr, b->y, stack_step(S, r, 0, final_norm));
+            linear(GemmArgs{b->x, l.wgu, b->act, nullptr, nullptr, n, 2 * l.ff, H, H, H, l.ff, 0, kActSiluMul}, l.sw_gu);
+            linear(GemmArgs{b->act, l.wd, b->y, nullptr, nullptr, n, H, l.ff, l.ff, l.ff, H, 0, kActNone}, l.sw_d);
+        }
+        norm(b->xr, b->y, stack_step(S, r, l.ff ? 1 : 0, final_norm));
+    }
+    GemmArgs ga{b->x, lm_head, b->logits, nullptr, nullptr, n, V, H, H, H, V, 0, kActNone};
+    ga.c_f32 = 1; ga.cap = S.c.logit_softcap;
+    linear(ga, sw_lm_head);
+    LMX_PROF("decode_batch.argmax");
+    launch_argmax_advance_batch(dt, b->logits, Vr, V, b->d_state_tab, nullptr, n, ids, embed, b->h, H, st, /*f32_logits=*/true);
+}
+
+void Model::stack_seq_copy(Seq* dst, const Seq* src, hipStream_t st) {
+    const size_t n = (size_t)src->len;
+    for (const StackRun& r : stk->runs) {
+        const StackLayer& l = stk->layers[(size_t)r.layer];
+        const size_t nk = (size_t)l.c.n_kv_heads;
+        LMX_CHECK_HIP(hipMemcpy2DAsync(dst->kc.as<char>() + r.kv_off, (size_t)s_max * l.D * es, src->kc.as<char>() + r.kv_off, (size_t)s_max * l.D * es, n * l.D * es, nk, hipMemcpyDeviceToDevice, st));
+        LMX_CHECK_HIP(hipMemcpy2DAsync(dst->vt.as<char>() + r.kv_off, (size_t)s_max * es, src->vt.as<char>() + r.kv_off, (size_t)s_max * es, n * es, nk * l.D, hipMemcpyDeviceToDevice, st));
+    }
+}
+
+}  // namespace lmx

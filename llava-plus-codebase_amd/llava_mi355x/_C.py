@@ -36,6 +36,17 @@ class LmxConfig(Structure):
     ]
 
 
+class LmxLayerConfig(Structure):
+    _fields_ = [("n_heads", c_int32), ("n_kv_heads", c_int32), ("qk_dim", c_int32), ("v_dim", c_int32), ("attn_scale", c_float), ("window", c_int32), ("softmax_sink", c_int32),
+                ("qk_norm", c_int32), ("qkv_bias", c_int32), ("out_gate", c_int32), ("rope_dims", c_int32), ("rope_table", c_int32), ("ff", c_int32), ("reserved", c_int32 * 8)]
+
+
+class LmxStackConfig(Structure):
+    _fields_ = [("abi_version", c_int32), ("dtype", c_int32), ("width", c_int32), ("vocab_size", c_int32), ("n_layers", c_int32), ("max_position", c_int32),
+                ("loop_start", c_int32), ("loop_stop", c_int32), ("loop_times", c_int32), ("norm_eps", c_float), ("residual_mult", c_float), ("logit_softcap", c_float),
+                ("gemm_variant", c_int32), ("reserved", c_int32 * 8)]
+
+
 def _load():
     # torch first: it preloads its bundled libamdhip64 / librccl by absolute path.  Our library must bind to THAT runtime
     # instance (same SONAMEs) — we share device pointers and streams with torch; loading the system copy first would put two
@@ -59,6 +70,12 @@ _SIGS = {
     "lmx_last_error": (c_char_p, []),
     "lmx_abi_version": (c_int32, []),
     "lmx_create": (c_int32, [POINTER(LmxConfig), POINTER(c_void_p)]),
+    "lmx_create_stack": (c_int32, [POINTER(LmxStackConfig), POINTER(LmxLayerConfig), POINTER(c_void_p)]),
+    "lmx_stack_set_rope": (c_int32, [c_void_p, c_int32, c_int32, c_void_p, c_int32]),
+    "lmx_row_pitch": (c_int32, [c_void_p]),
+    "lmx_vocab_pitch": (c_int32, [c_void_p]),
+    "lmx_logit_dtype": (c_int32, [c_void_p]),
+    "lmx_layer_runs": (c_int32, [c_void_p]),
     "lmx_destroy": (c_int32, [c_void_p]),
     "lmx_load_weight": (c_int32, [c_void_p, c_char_p, c_void_p, c_int32, c_int32, _i64p, c_void_p]),
     "lmx_finalize_weights": (c_int32, [c_void_p]),
@@ -138,6 +155,7 @@ _SIGS = {
     "lmx_op_embed_bwd": (c_int32, [c_int32, c_void_p, c_void_p, c_void_p, c_void_p, c_int32, c_int32, c_void_p]),
     "lmx_op_sumsq": (c_int32, [c_int32, c_void_p, c_int64, c_void_p, c_void_p]),
     "lmx_prefill_batch": (c_int32, [c_void_p, c_void_p, c_int32, c_void_p, c_void_p, c_int32, c_int32, c_void_p]),
+    "lmx_prefill_batch_logits": (c_int32, [c_void_p, c_void_p, c_int32, c_void_p, c_void_p, c_int32, c_void_p, c_void_p, c_void_p, c_int32, c_void_p]),
     "lmx_seq_copy": (c_int32, [c_void_p, c_void_p, c_void_p]),
     "lmx_seq_truncate": (c_int32, [c_void_p, c_int32, c_void_p]),
     "lmx_op_hash128": (c_int32, [c_void_p, ctypes.c_uint64, c_int32, c_void_p, c_void_p]),

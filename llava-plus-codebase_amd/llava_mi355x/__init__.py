@@ -11,6 +11,12 @@ def __getattr__(name):
     if name in ("LlavaConfig", "LlavaLlamaForCausalLM", "LlavaLlamaModel", "LmxKVCache"):
         from . import model
         return getattr(model, name)
+    if name in ("SiteraxConfig", "SiteraxForCausalLM"):
+        from . import siterax
+        return getattr(siterax, name)
+    if name == "load_model":
+        from .registry import load_model
+        return load_model
     if name == "load_pretrained_model":
         from .builder import load_pretrained_model
         return load_pretrained_model

@@ -76,8 +76,8 @@ def beam_search(model, ids: torch.Tensor, images, attention_mask, num_beams: int
     and finalize() ranks the open beams with the finished hypotheses.
     sample: None = beam search; dict(temperature, top_p, top_k, seed) = beam sample (see the module docstring)."""
     from .batching import DecodeBatch
-    from .model import LmxKVCache
-    B, dev, dt = int(num_beams), model.device, model.dtype
+    from .engine_lm import LmxKVCache
+    B, dev, dt = int(num_beams), model.device, model.logits_dtype
     V, Vpitch = model.config.vocab_size, model._vocab_cap
     K = 2 * B
     cache0, logits0 = model._prefill_request(ids, images, attention_mask, None, prefill_chunk, return_logits=True)

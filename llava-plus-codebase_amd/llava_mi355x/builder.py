@@ -10,36 +10,14 @@ layouts).  Out of scope, raise NotImplementedError: 8-bit/4-bit (bitsandbytes), 
 """
 from __future__ import annotations
 
-import glob
 import os
-from typing import Iterator, Optional, Tuple
+from typing import Optional
 
 import torch
 
 from .constants import DEFAULT_IM_END_TOKEN, DEFAULT_IM_START_TOKEN, DEFAULT_IMAGE_PATCH_TOKEN
 from .model import LlavaConfig, LlavaLlamaForCausalLM
-
-
-def iter_checkpoint(path: str) -> Iterator[Tuple[str, torch.Tensor]]:
-    """Yield (key, tensor) from every weight shard in a HF-format directory (or a single file)."""
-    files = [path] if os.path.isfile(path) else sorted(glob.glob(os.path.join(path, "*.safetensors")))
-    if not files:
-        files = sorted(glob.glob(os.path.join(path, "pytorch_model*.bin")))
-    if not files:
-        raise FileNotFoundError(f"no *.safetensors / pytorch_model*.bin under {path}")
-    for f in files:
-        if f.endswith(".safetensors"):
-            from safetensors import safe_open
-            with safe_open(f, framework="pt", device="cpu") as sf:
-                for k in sf.keys():
-                    yield k, sf.get_tensor(k)
-        else:
-            try:
-                sd = torch.load(f, map_location="cpu", mmap=True, weights_only=True)
-            except (RuntimeError, ValueError):          # legacy (non-zip) .bin shards cannot be memory-mapped; the reference loads them too
-                sd = torch.load(f, map_location="cpu", weights_only=True)
-            for k, v in sd.items():
-                yield k, v
+from .registry import family_of, iter_checkpoint
 
 
 def read_lora_adapter(model_path: str):
@@ -156,12 +134,45 @@ def from_pretrained(model_path, config: Optional[LlavaConfig] = None, torch_dtyp
     return model
 
 
+def _load_text_model(family, model_path, device, torch_dtype, max_position):
+    """A text-only family of the registry behind the same 4-tuple: (tokenizer or None, model, None, context_len); the batching and reuse switches apply as below."""
+    tokenizer = None
+    if any(os.path.isfile(os.path.join(model_path, n)) for n in ("tokenizer.json", "tokenizer.model", "tokenizer_config.json")):
+        from transformers import AutoTokenizer
+        tokenizer = AutoTokenizer.from_pretrained(model_path, use_fast=False)
+    model = family.load(model_path, torch_dtype=torch_dtype, device=device, max_position=max_position)
+    _serving_switches(model)
+    return tokenizer, model, None, model.s_max
+
+
+def _serving_switches(model) -> None:
+    # continuous batching for model_worker's thread-per-request serving (llava/serve/model_worker.py:174-185): opt-in by env so the
+    # reference's call signature stays untouched.  LLAVA_MI355X_BATCH=<capacity> (e.g. 32)
+    cap = int(os.environ.get("LLAVA_MI355X_BATCH", "0") or 0)
+    if cap > 1:
+        # LLAVA_MI355X_PACKED_PREFILL=0: prefills stay on the request threads (one at a time) instead of being packed by the scheduler
+        model.enable_batching(capacity=cap, packed_prefill=os.environ.get("LLAVA_MI355X_PACKED_PREFILL", "1") != "0")
+    # reuse between the turns of a conversation (the LLaVA-Plus tool loop re-sends image + first exchange: gradio_web_server_llava_plus.py:600-637), opt-in:
+    # LLAVA_MI355X_REUSE=1 or "<images>,<prefixes>" (reuse.py: image features by pixel content, KV prefixes of finished requests)
+    ru = os.environ.get("LLAVA_MI355X_REUSE", "0") or "0"
+    if ru != "0":
+        parts = [int(v) for v in ru.split(",")] if "," in ru else []
+        model.enable_reuse(images=parts[0] if parts else 64, prefixes=parts[1] if len(parts) > 1 else 32)
+
+
 def load_pretrained_model(model_path, model_base, model_name, load_8bit=False, load_4bit=False, device_map="auto", device="cuda",
                           torch_dtype: Optional[torch.dtype] = None, tp_rank: int = 0, tp_world: int = 1, max_position: Optional[int] = None):
     """Same steps, in the same order, as llava/model/builder.py:26-151 for the LLaVA / LLaMA family."""
     if load_8bit or load_4bit:
         raise NotImplementedError("bitsandbytes 8-bit/4-bit loading is CUDA-only and out of scope of the MI355X path")
     name_l = model_name.lower()
+    if model_base is None and "lora" not in name_l and os.path.isfile(os.path.join(model_path, "config.json")):
+        try:
+            family = family_of(model_path)
+        except ValueError:
+            family = None
+        if family is not None and not family.multimodal:
+            return _load_text_model(family, model_path, device, torch_dtype, max_position)
     if "mpt" in name_l:
         raise NotImplementedError("MPT checkpoints are not supported by the MI355X path (LLaMA/Vicuna family only)")
     if "llava" not in name_l:
@@ -204,18 +215,7 @@ def load_pretrained_model(model_path, model_base, model_name, load_8bit=False, l
     vision_tower.to(device=device, dtype=torch.float16)
     image_processor = vision_tower.image_processor
     model.finalize_weights()
-    # continuous batching for model_worker's thread-per-request serving (llava/serve/model_worker.py:174-185): opt-in by env so the
-    # reference's call signature stays untouched.  LLAVA_MI355X_BATCH=<capacity> (e.g. 32)
-    cap = int(os.environ.get("LLAVA_MI355X_BATCH", "0") or 0)
-    if cap > 1:
-        # LLAVA_MI355X_PACKED_PREFILL=0: prefills stay on the request threads (one at a time) instead of being packed by the scheduler
-        model.enable_batching(capacity=cap, packed_prefill=os.environ.get("LLAVA_MI355X_PACKED_PREFILL", "1") != "0")
-    # reuse between the turns of a conversation (the LLaVA-Plus tool loop re-sends image + first exchange: gradio_web_server_llava_plus.py:600-637), opt-in:
-    # LLAVA_MI355X_REUSE=1 or "<images>,<prefixes>" (reuse.py: image features by pixel content, KV prefixes of finished requests)
-    ru = os.environ.get("LLAVA_MI355X_REUSE", "0") or "0"
-    if ru != "0":
-        parts = [int(v) for v in ru.split(",")] if "," in ru else []
-        model.enable_reuse(images=parts[0] if parts else 64, prefixes=parts[1] if len(parts) > 1 else 32)
+    _serving_switches(model)
     from . import mm_utils
     mm_utils.set_device_preprocess_model(model)          # used by process_images when LLAVA_MI355X_DEVICE_PREPROCESS=1
     context_len = getattr(model.config, "max_sequence_length", 2048)     # builder.py:146-149
