@@ -61,10 +61,11 @@ def parse():
     ap.add_argument("--train-keep-gb", type=float, default=-1.0, help="config5: bytes of layer activations kept instead of recomputed (GB; < 0 = what 88 %% of the device "
                                                                       "memory leaves after a fully recomputing step, 0 = recompute every layer as the reference's gradient_checkpointing)")
     ap.add_argument("--train-seq", type=int, default=1024, help="config5: positions per sample after the image splice (the reference caps at 2048)")
-    ap.add_argument("--workload", default="config2", choices=["config2", "config3", "config5"],
+    ap.add_argument("--workload", default="config2", choices=["config2", "config3", "config5", "siterax"],
                     help="config2 (default, BASELINE metric): one request, batch 1.  config3: LLaVA-1.5-13B geometry, 8 requests (8 images), "
                          "chunked prefill (512 rows), the 8 sequences decode together; prefill and decode reported separately.  config5: one "
-                         "visual-instruction-tuning step (forward, backward, AdamW, ZeRO-2 over the ranks) of LLaVA-1.5-7B geometry")
+                         "visual-instruction-tuning step (forward, backward, AdamW, ZeRO-2 over the ranks) of LLaVA-1.5-7B geometry.  siterax: prefill and decode of "
+                         "the Siterax decoder at real layer sizes beside the LLaMA decoder at equal size, with per-kernel roofline fractions (one GPU)")
     ap.add_argument("--no-parity-probe", action="store_true", help="skip the live parity probe (the fp32 verification engine on the same bf16-rounded weights: "
                                                                   "last-position prefill logits and the first greedy ids of the timed request)")
     ap.add_argument("--no-pmc", action="store_true", help="skip the rocprofv3 --pmc passes that measure roofline.traffic")
@@ -765,6 +766,171 @@ def run_config3(a, model, cfg, synth, dev, dtype, barrier, world, rank, share, b
         dist.destroy_process_group()
 
 
+# ---- Siterax beside the LLaMA decoder ---------------------------------------------------------------------------------------------------------
+# name -> (width, heads, kv heads, head width, ff, layers, vocab, window); window 0 = every key (the like-for-like row), otherwise what a windowed model would use
+SITERAX_SIZES = {
+    "w2048": (2048, 16, 4, 128, 5632, 12, 32000, 0),
+    "w4096": (4096, 32, 8, 128, 11008, 12, 32000, 0),
+    "w4096_win1024": (4096, 32, 8, 128, 11008, 12, 32000, 1024),
+    "w3072_d96": (3072, 32, 8, 96, 8192, 12, 32000, 0),
+}
+
+
+def _random_weights(model, shapes, dev, dtype, seed=0):
+    g = torch.Generator(device=dev).manual_seed(seed)
+    for name, shape in shapes:
+        t = torch.randn(shape, generator=g, device=dev, dtype=torch.float32)
+        model.load_tensor(name, (1 + 0.1 * t if len(shape) == 1 and "norm" in name else t / shape[-1] ** 0.5).to(dtype))
+    model.finalize_weights()
+    return model
+
+
+def _siterax_model(size, dev, dtype, max_position, loop=None):
+    from llava_mi355x.siterax import SiteraxConfig, SiteraxForCausalLM
+    W, H, G, D, F, L, V, win = size
+    layer = {"type": "attention", "mixer": {"heads": H, "kv_heads": G, "dim": D, "vdim": D, "scale": D ** -0.5, "mask": {"size": win} if win else None,
+                                            "rot": {"dims": D, "base": 10000.0, "scaling": {"factor": 1.0}}}, "mlp": {"kind": "dense", "ff": F}}
+    c = SiteraxConfig.from_dict({"vocab": V, "width": W, "layers": [layer] * L, "norm": {"eps": 1e-5}, "residual_mult": 0.5, "logit_softcap": 30.0, "loop": loop})
+    shapes = [("embed", (V, W)), ("head", (V, W)), ("final.norm", (W,))]
+    for i in range(L):
+        p = f"l{i}."
+        shapes += [(p + n, (W,)) for n in ("norm1", "norm1b", "norm2", "norm2b")]
+        shapes += [(p + "mix.q", (H * D, W)), (p + "mix.k", (G * D, W)), (p + "mix.v", (G * D, W)), (p + "mix.q.b", (H * D,)), (p + "mix.k.b", (G * D,)), (p + "mix.v.b", (G * D,)),
+                   (p + "mix.q.norm", (D,)), (p + "mix.k.norm", (D,)), (p + "mix.g", (H, W)), (p + "mix.o", (W, H * D)),
+                   (p + "mlp.gate", (F, W)), (p + "mlp.up", (F, W)), (p + "mlp.down", (W, F))]
+    return _random_weights(SiteraxForCausalLM(c, dtype=dtype, device=dev, max_position=max_position), shapes, dev, dtype)
+
+
+def _llama_model(size, dev, dtype, max_position):
+    from llava_mi355x.model import LlavaConfig, LlavaLlamaForCausalLM
+    W, H, G, D, F, L, V, _ = size
+    H, G = (H, G) if W == H * 128 else (W // 128, max(1, W // 128 * G // H))          # the LLaMA decoder has head widths 64 / 128: the same width in heads of 128
+    c = LlavaConfig(hidden_size=W, intermediate_size=F, num_hidden_layers=L, num_attention_heads=H, num_key_value_heads=G, vocab_size=V, max_position_embeddings=max_position)
+    shapes = [("model.embed_tokens.weight", (V, W)), ("lm_head.weight", (V, W)), ("model.norm.weight", (W,))]
+    for i in range(L):
+        p = f"model.layers.{i}."
+        shapes += [(p + "input_layernorm.weight", (W,)), (p + "post_attention_layernorm.weight", (W,)), (p + "self_attn.q_proj.weight", (W, W)),
+                   (p + "self_attn.k_proj.weight", (G * 128, W)), (p + "self_attn.v_proj.weight", (G * 128, W)), (p + "self_attn.o_proj.weight", (W, W)),
+                   (p + "mlp.gate_proj.weight", (F, W)), (p + "mlp.up_proj.weight", (F, W)), (p + "mlp.down_proj.weight", (W, F))]
+    return _random_weights(LlavaLlamaForCausalLM(c, None, dtype=dtype, device=dev, max_position=max_position), shapes, dev, dtype), H, G, 128
+
+
+def _kernel_rooflines(prof, size, geom, T, ctx, n_batch):
+    """Per in-situ kernel group: average us and the fraction of its own roofline (MFMA flops or HBM bytes, whichever bounds it) at these sizes."""
+    W, _, _, _, F, L, V, win = size
+    H, G, D = geom
+    qkv = (H + 2 * G) * D
+    seen = sum(min(i + 1, win) if win else i + 1 for i in range(T))
+    keys = min(ctx, win) if win else ctx
+    mfma = lambda fl: fl / (PEAK_BF16_TFLOPS * 1e12)
+    hbm = lambda by: by / (PEAK_HBM_GBS * 1e9)
+    floor = {"prefill.gemm.qkv": mfma(2.0 * T * W * qkv), "prefill.gemm.o": mfma(2.0 * T * W * H * D), "prefill.gemm.gate_up": mfma(4.0 * T * W * F),
+             "prefill.gemm.down": mfma(2.0 * T * W * F), "prefill.attn": mfma(4.0 * seen * H * D), "prefill.rmsnorm": hbm(4.0 * T * W), "prefill.residual_norm": hbm(14.0 * T * W),
+             "prefill.rope_kv": hbm(4.0 * T * qkv), "prefill.norm_rope_kv": hbm(4.0 * T * qkv),
+             "decode.gemv.qkv": hbm(2.0 * W * qkv), "decode.gemv.o": hbm(2.0 * W * H * D), "decode.gemv.gate_up": hbm(4.0 * W * F), "decode.gemv.down": hbm(2.0 * W * F),
+             "decode.gemv.lm_head": hbm(2.0 * W * V), "decode.attn": hbm(4.0 * keys * G * D), "decode_batch.attn": hbm(4.0 * keys * G * D * n_batch)}
+    out = {}
+    for k, (ms, n) in sorted(prof.items()):
+        us = ms * 1e3 / max(1, n)
+        out[k] = {"us": round(us, 2), "launches": n, **({"roofline_frac": round(floor[k] * 1e6 / us, 3)} if k in floor and us > 0 else {})}
+    return out
+
+
+def _time_decoder(model, T, ctx, new_tokens, steps, warmup, batches=(8, 32)):
+    """Prefill of T rows, `new_tokens` greedy tokens at context ctx, batched decode steps: medians over `steps` timed repetitions."""
+    import ctypes
+    import statistics
+    from llava_mi355x._C import check, lib, ptr, stream_handle
+    from llava_mi355x.batching import DecodeBatch
+    from llava_mi355x.engine_lm import LmxKVCache
+    ids = torch.randint(0, model.config.vocab_size, (1, max(T, ctx)), device=model.device)
+    emb = model.get_model().embed_tokens(ids)[0].contiguous()
+
+    def prefill(rows):
+        c = LmxKVCache(model, 1)
+        check(lib.lmx_prefill(model._h, c.seqs[0], ptr(emb), rows, 0, None, 0, 1, stream_handle()), "lmx_prefill")
+        return c
+
+    def timed(fn):
+        torch.cuda.synchronize()
+        t0 = time.perf_counter()
+        r = fn()
+        torch.cuda.synchronize()
+        return time.perf_counter() - t0, r
+    pre, dec = [], []
+    for it in range(warmup + steps):
+        dt, c = timed(lambda: prefill(T))
+        c.close()
+        c = prefill(ctx)
+        dd, _ = timed(lambda: check(lib.lmx_decode(model._h, c.seqs[0], -1, new_tokens, None, 1, stream_handle()), "lmx_decode"))
+        c.close()
+        if it >= warmup:
+            pre.append(dt); dec.append(dd / new_tokens)
+    out = {"prefill_tok_s": round(T / statistics.median(pre), 1), "prefill_ms": round(statistics.median(pre) * 1e3, 3), "decode_tok_s": round(1 / statistics.median(dec), 1),
+           "decode_ms": round(statistics.median(dec) * 1e3, 4)}
+    for n in batches:
+        cs = [prefill(ctx // 2) for _ in range(n)]
+        b = DecodeBatch(model, n)
+        ts = []
+        for it in range(warmup + steps):
+            dt, _ = timed(lambda: b.step([c.seqs[0] for c in cs], None, 16, True, want_ids=False))
+            if it >= warmup:
+                ts.append(dt / 16)
+        out[f"decode_batch{n}_tok_s"] = round(n / statistics.median(ts), 1)
+        b.close()
+        for c in cs:
+            c.close()
+    c = prefill(ctx)
+    model.profile(True)
+    prefill(T).close()
+    check(lib.lmx_decode(model._h, c.seqs[0], -1, 8, None, 1, stream_handle()), "lmx_decode")
+    prof = model.profile_read()
+    model.profile(False)
+    n = batches[-1]
+    cs = [prefill(ctx // 2) for _ in range(n)]
+    model.profile(True)
+    b = DecodeBatch(model, n)
+    b.step([x.seqs[0] for x in cs], None, 4, True, want_ids=False)
+    batch_prof = {k: v for k, v in model.profile_read().items() if k.startswith("decode_batch")}
+    model.profile(False)
+    b.close()
+    for x in cs + [c]:
+        x.close()
+    return out, prof, batch_prof
+
+
+def run_siterax(a, dev):
+    dtype = {"bf16": torch.bfloat16, "f16": torch.float16}[a.dtype]
+    T, ctx, new = 2048, 2048, 64
+    rows, first = {}, None
+    for name, size in SITERAX_SIZES.items():
+        W, H, G, D = size[:4]
+        res = {}
+        for kind in ("siterax", "llama"):
+            if kind == "siterax":
+                model, geom = _siterax_model(size, dev, dtype, 4096), (H, G, D)
+            else:
+                model, h, g, d = _llama_model(size, dev, dtype, 4096)
+                geom = (h, g, d)
+            fig, prof, bprof = _time_decoder(model, T, ctx, new, a.steps, a.warmup)
+            sz = size if kind == "siterax" else size[:7] + (0,)
+            fig["kernels"] = _kernel_rooflines({k: v for k, v in prof.items()}, sz, geom, T, ctx, 1)
+            fig["kernels"].update(_kernel_rooflines(bprof, sz, geom, T, ctx // 2, 32))
+            res[kind] = fig
+            del model
+            torch.cuda.empty_cache()
+        res["prefill_ratio"] = round(res["siterax"]["prefill_tok_s"] / res["llama"]["prefill_tok_s"], 3)
+        res["decode_ratio"] = round(res["siterax"]["decode_tok_s"] / res["llama"]["decode_tok_s"], 3)
+        rows[name] = res
+        first = first or res
+        print(f"# {name}: prefill {res['prefill_ratio']} x, decode {res['decode_ratio']} x the LLaMA decoder", file=sys.stderr, flush=True)
+    print(json.dumps({"metric": "siterax_decode_tokens_per_s", "value": first["siterax"]["decode_tok_s"], "unit": "tok/s", "n_gpus": 1, "steps": a.steps, "warmup": a.warmup,
+                      "ms_per_step": first["siterax"]["decode_ms"], "higher_is_better": True, "scaling": "weak", "vs_baseline": None, "dtype": a.dtype, "data": "synthetic (random weights)",
+                      "config": {"workload": f"siterax: prefill of {T} rows, {new} greedy tokens at context {ctx}, decode batches of 8 and 32 at context {ctx // 2}",
+                                 "sizes": {k: dict(zip(("width", "heads", "kv_heads", "dim", "ff", "layers", "vocab", "window"), v)) for k, v in SITERAX_SIZES.items()}},
+                      "rows": rows}), flush=True)
+
+
 def main():
     a = parse()
     world = int(os.environ.get("WORLD_SIZE", "1"))
@@ -786,6 +952,10 @@ def main():
             dist.init_process_group("gloo")
         else:
             dist.init_process_group("nccl", device_id=dev)
+
+    if a.workload == "siterax":
+        run_siterax(a, dev)
+        return
 
     from synthetic import build as harness, recipes as synth
     if a.workload == "config3":

@@ -405,6 +405,7 @@ int lmx_model_set_option(lmx_model* m, const char* key, int32_t value) {
     if (k == "fuse_rope") m->impl.opt_fuse_rope = value != 0;
     else if (k == "vis_pack") m->impl.opt_vis_pack = value != 0;
     else if (k == "decode_splitq") m->impl.opt_splitq = value != 0;
+    else if (k == "stack_fuse") m->impl.opt_stack_fuse = value != 0;
     else if (k == "debug_splitq_timeout") m->impl.debug_splitq_timeout = value;
     else throw Error{"lmx_model_set_option: unknown option '" + k + "'"};
     LMX_API_END

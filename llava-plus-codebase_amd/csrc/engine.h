@@ -183,6 +183,7 @@ struct Model {
     // vis_pack:  CLIP K / V^T pack in the tower's q|k|v GEMM epilogue instead of a pack launch — bit-identical, launch count
     // splitq:    the decode step's q|k|v projection as q-launch + (k|v projection ∥ attention) launch (decode_attn.hip) — bit-identical
     bool opt_fuse_rope = true, opt_vis_pack = true, opt_splitq = true;
+    bool opt_stack_fuse = true;         // stack_fuse: a layer-stack decode step's residual addition and norms inside the linear's launch (equal up to rounding)
     // Sequences in existence (lmx_seq_create .. lmx_seq_destroy).  The split-q launch parks one waiting workgroup per head until its own launch's projection has
     // run; launches of DIFFERENT sequences (request threads on their own streams) may be resident together, so the form is only taken while all sequences'
     // waiters together (live_seqs x heads) fill at most half of the chip's ~1024 workgroup slots — the projection's workgroups then always find a slot

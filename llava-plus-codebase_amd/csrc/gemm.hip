@@ -630,6 +630,14 @@ __global__ __launch_bounds__(256) void gemv2_kernel(GemvArgs a) {
     gemv2_body<T, R, P, GEMV2_NX, false>(a, (int)blockIdx.x, smem, nullptr, 0u);
 }
 
+// the same linear on a row that is formed in front of it: residual addition and both norms of the layer-stack decoders (gemv2.h RES).  The last workgroup stores x'.
+template <typename T, int R, int P, int GEMV2_NX>
+__global__ __launch_bounds__(256) void gemv2_res_kernel(GemvArgs a, ResidualNormArgs rn) {
+    extern __shared__ __attribute__((aligned(16))) char smem[];
+    if (blockIdx.x == gridDim.x - 1) { residual_row_store<T>(rn, reinterpret_cast<float*>(smem)); return; }
+    gemv2_body<T, R, P, GEMV2_NX, false, true>(a, (int)blockIdx.x, smem, nullptr, 0u, nullptr, &rn);
+}
+
 // ---------------------------------------------------------------------------------------------
 // host launchers
 // ---------------------------------------------------------------------------------------------
@@ -789,6 +797,34 @@ bool gemv2_applies(int dtype, const GemvArgs& a) {
     if (dtype != kBF16 && dtype != kF16) return false;
     if (((size_t)a.ldw * 2) % 16 != 0 || (size_t)a.N * a.ldw * 2 >= ((size_t)1 << 32)) return false;
     return a.K <= 16384 && reinterpret_cast<uintptr_t>(a.X) % 16 == 0;
+}
+
+template <typename T, int R, int P, int NX>
+static void launch_gemv2_res_rx(const GemvArgs& a, const ResidualNormArgs& rn, hipStream_t st) {
+    auto kern = gemv2_res_kernel<T, R, P, NX>;
+    static bool attr_set = false;
+    if (!attr_set) { LMX_CHECK_HIP(hipFuncSetAttribute(reinterpret_cast<const void*>(kern), hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024)); attr_set = true; }
+    LMX_LAUNCH(kern, dim3(cdiv(a.N, 4 * R) + 1), dim3(256), gemv2_smem_bytes(a.K, (int)sizeof(T)), st, a, rn);
+    LMX_CHECK_HIP(hipGetLastError());
+}
+template <typename T>
+static void launch_gemv2_res(const GemvArgs& a, const ResidualNormArgs& rn, hipStream_t st) {
+    if (a.K <= 2048) launch_gemv2_res_rx<T, 2, 4, 1>(a, rn, st);
+    else if (a.K <= 4096) launch_gemv2_res_rx<T, 2, 4, 2>(a, rn, st);
+    else launch_gemv2_res_rx<T, 2, 4, 4>(a, rn, st);
+}
+
+bool gemv_residual_applies(int dtype, const GemvArgs& a) {
+    if (dtype != kBF16 && dtype != kF16) return false;
+    if (((size_t)a.ldw * 2) % 16 != 0 || (size_t)a.N * a.ldw * 2 >= ((size_t)1 << 32)) return false;
+    return a.K % 8 == 0 && a.K <= 8192;
+}
+void launch_gemv_residual(int dtype, GemvArgs a, const ResidualNormArgs& rn, hipStream_t st) {
+    LMX_REQUIRE(gemv_residual_applies(dtype, a), "gemv_residual: 16-bit weights, 16-byte rows, K up to 8192");
+    LMX_REQUIRE(rn.H == a.K && rn.pre_w && rn.x_out && rn.x_out != rn.x_in && (!rn.y || rn.post_w) && (rn.y || rn.inject || rn.x_in), "gemv_residual: bad residual arguments (x_out must be another row than x_in)");
+    LMX_REQUIRE(!a.R && (a.act != kActSiluMul || a.N % 64 == 0), "gemv_residual: no second residual; SiLU*mul needs N % 64 == 0");
+    a.X = rn.y; a.norm_w = rn.pre_w;
+    if (dtype == kBF16) launch_gemv2_res<bf16_t>(a, rn, st); else launch_gemv2_res<f16_t>(a, rn, st);
 }
 
 // The single-row decode linears of 16-bit models take the hand-counted stream.  (R rows per wave, P rounds in flight) per shape from the in-situ sweep

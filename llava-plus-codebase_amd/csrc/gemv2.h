@@ -18,8 +18,12 @@ namespace lmx {
 
 constexpr size_t gemv2_smem_bytes(int K, int es) { return (size_t)K * es + 16; }
 
-template <typename T, int R, int P, int GEMV2_NX, bool PUBLISH>
-__device__ __forceinline__ void gemv2_body(const GemvArgs& a, int bid, char* smem, unsigned long long* gran, unsigned tag, unsigned long long* ts = nullptr) {
+// RES (the layer-stack decoders' linears): the input row is not a stored vector but what residual_norm_kernel (stack_ops.hip) would have written — xn = rms_norm(x') pre_w with
+// x' = x_in + mult rms_norm(y) post_w + inject, y = a.X — computed by every workgroup while its first weight rounds are on the wire; one workgroup past the linear's own
+// (residual_row_store) stores x' for the launches that follow, so nobody stores inside the counted stream.
+template <typename T, int R, int P, int GEMV2_NX, bool PUBLISH, bool RES = false>
+__device__ __forceinline__ void gemv2_body(const GemvArgs& a, int bid, char* smem, unsigned long long* gran, unsigned tag, unsigned long long* ts = nullptr,
+                                           const ResidualNormArgs* rn = nullptr) {
     if (ts && threadIdx.x == 0 && (bid & 31) == 0) __hip_atomic_fetch_min(ts + 6, (unsigned long long)__builtin_amdgcn_s_memrealtime(), __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);      // debug timeline (decode_attn.hip)
     static_assert(sizeof(T) == 2, "gemv2: 16-bit weights");
     T* xs = reinterpret_cast<T*>(smem);                       // [K]
@@ -55,12 +59,28 @@ __device__ __forceinline__ void gemv2_body(const GemvArgs& a, int bid, char* sme
     // ---- x (one short row, L2-resident) is requested ahead of the weights, in the same counted queue: it lands first and is staged / normalised while
     //      the first P weight rounds are still on the wire.  (As plain loads behind the weight issue its wait was a vmcnt(0): staging started only after
     //      the first P rounds had landed too.)
-    const ws_v4i rsX = ws_make_rsrc(a.X, 0x7fffffffu);
+    const bool has_x = !RES || a.X != nullptr;                // RES: the first linear of a step has no sublayer output in front of it
+    const ws_v4i rsX = ws_make_rsrc(has_x ? a.X : a.W, 0x7fffffffu);
     ws_u32x4 xraw[GEMV2_NX];
+    if (has_x) {
 #pragma unroll
-    for (int i = 0; i < GEMV2_NX; ++i) {
-        const int c = tid + 256 * i;
-        if (c < KC) ws_load_plain(xraw[i], (uint32_t)c * 16u, rsX, 0u);
+        for (int i = 0; i < GEMV2_NX; ++i) {
+            const int c = tid + 256 * i;
+            if (c < KC) ws_load_plain(xraw[i], (uint32_t)c * 16u, rsX, 0u);
+        }
+    }
+    ws_u32x4 praw[RES ? GEMV2_NX : 1], iraw[RES ? GEMV2_NX : 1], r0raw[RES ? GEMV2_NX : 1], r1raw[RES ? GEMV2_NX : 1];
+    if constexpr (RES) {
+        const ws_v4i rsP = ws_make_rsrc(has_x ? rn->post_w : a.W, 0x7fffffffu), rsI = ws_make_rsrc(rn->inject ? rn->inject : a.W, 0x7fffffffu),
+                     rsR0 = ws_make_rsrc(rn->x_in ? static_cast<const void*>(rn->x_in) : a.W, 0x7fffffffu);
+#pragma unroll
+        for (int i = 0; i < GEMV2_NX; ++i) {
+            const int c = tid + 256 * i;
+            if (c >= KC) continue;
+            if (has_x) ws_load_plain(praw[i], (uint32_t)c * 16u, rsP, 0u);
+            if (rn->inject) ws_load_plain(iraw[i], (uint32_t)c * 16u, rsI, 0u);
+            if (rn->x_in) { ws_load_plain(r0raw[i], (uint32_t)c * 32u, rsR0, 0u); ws_load_plain(r1raw[i], (uint32_t)c * 32u + 16u, rsR0, 0u); }
+        }
     }
     const ws_v4i rsG = ws_make_rsrc(a.norm_w ? a.norm_w : a.W, 0x7fffffffu);
     ws_u32x4 graw[GEMV2_NX];                                  // RMSNorm weights of the same chunks (same queue position: older than every weight load)
@@ -85,7 +105,66 @@ __device__ __forceinline__ void gemv2_body(const GemvArgs& a, int bid, char* sme
 
     // ---- stage x into LDS: plain copy | RMS-normalised (gemv_kernel's arithmetic; x is read from memory ONCE: the chunks go to LDS raw, the statistics
     //      are taken on the way, and each thread normalises in place the chunks it wrote itself — no second global round trip behind the weight loads) ------
-    {
+    if constexpr (RES) {
+        float xv[GEMV2_NX][8];
+        const float rH = 1.f / (float)rn->H_real;
+        float inv1 = 0.f;
+        if (has_x) {
+            float ss = 0.f;
+#pragma unroll
+            for (int i = 0; i < GEMV2_NX; ++i) {
+                const int c = tid + 256 * i;
+                if (c < KC) {
+                    ws_wait1<P * R>(xraw[i]);
+                    float v[8]; ws_unpack8<T>(xraw[i], v);
+#pragma unroll
+                    for (int e = 0; e < 8; ++e) ss += v[e] * v[e];
+                }
+            }
+            inv1 = rn->mult / sqrtf(block_sum<4>(ss, red) * rH + rn->eps);
+        }
+        float s2 = 0.f;
+#pragma unroll
+        for (int i = 0; i < GEMV2_NX; ++i) {
+            const int c = tid + 256 * i;
+            if (c < KC) {
+#pragma unroll
+                for (int e = 0; e < 8; ++e) xv[i][e] = 0.f;
+                if (rn->x_in) {
+                    ws_wait1<P * R>(r0raw[i]); ws_wait1<P * R>(r1raw[i]);
+#pragma unroll
+                    for (int e = 0; e < 4; ++e) { xv[i][e] = __uint_as_float(r0raw[i][e]); xv[i][4 + e] = __uint_as_float(r1raw[i][e]); }
+                }
+                if (has_x) {
+                    float v[8], g[8];
+                    ws_unpack8<T>(xraw[i], v);
+                    ws_wait1<P * R>(praw[i]); ws_unpack8<T>(praw[i], g);
+#pragma unroll
+                    for (int e = 0; e < 8; ++e) xv[i][e] += v[e] * inv1 * g[e];
+                }
+                if (rn->inject) {
+                    float g[8];
+                    ws_wait1<P * R>(iraw[i]); ws_unpack8<T>(iraw[i], g);
+#pragma unroll
+                    for (int e = 0; e < 8; ++e) xv[i][e] += g[e];
+                }
+#pragma unroll
+                for (int e = 0; e < 8; ++e) s2 += xv[i][e] * xv[i][e];
+            }
+        }
+        const float inv2 = 1.f / sqrtf(block_sum<4>(s2, red) * rH + rn->eps);
+#pragma unroll
+        for (int i = 0; i < GEMV2_NX; ++i) {
+            const int c = tid + 256 * i;
+            if (c < KC) {
+                float g[8];
+                ws_wait1<P * R>(graw[i]); ws_unpack8<T>(graw[i], g);
+#pragma unroll
+                for (int e = 0; e < 8; ++e) xv[i][e] = xv[i][e] * inv2 * g[e];
+                store8<T>(xs + c * 8, xv[i]);
+            }
+        }
+    } else {
         const T* g = reinterpret_cast<const T*>(a.norm_w);
         float ss = 0.f;
 #pragma unroll
@@ -184,6 +263,44 @@ __device__ __forceinline__ void gemv2_body(const GemvArgs& a, int bid, char* sme
             if (ts && (bid & 31) == 31 && r == 0) __hip_atomic_fetch_max(ts + 7, (unsigned long long)__builtin_amdgcn_s_memrealtime(), __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
         } else if (a.c_f32) reinterpret_cast<float*>(a.C)[n] = soft_cap(v, a.cap);
         else C[n] = from_f32<T>(v);
+    }
+}
+
+// x' of one row to rn.x_out by the 256 threads of the calling workgroup (see RES above)
+template <typename T>
+__device__ __forceinline__ void residual_row_store(const ResidualNormArgs& rn, float* red) {
+    const T* y = reinterpret_cast<const T*>(rn.y);
+    const T* post = reinterpret_cast<const T*>(rn.post_w);
+    const T* inj = reinterpret_cast<const T*>(rn.inject);
+    const int HC = rn.H >> 3, tid = threadIdx.x;
+    float inv1 = 0.f;
+    if (y) {
+        float ss = 0.f;
+        for (int c = tid; c < HC; c += 256) {
+            float v[8]; load8<T>(y + c * 8, v);
+#pragma unroll
+            for (int e = 0; e < 8; ++e) ss += v[e] * v[e];
+        }
+        inv1 = rn.mult / sqrtf(block_sum<4>(ss, red) * (1.f / (float)rn.H_real) + rn.eps);
+    }
+    for (int c = tid; c < HC; c += 256) {
+        float x[8], v[8], g[8];
+        if (rn.x_in) load8<float>(rn.x_in + c * 8, x);
+        else {
+#pragma unroll
+            for (int e = 0; e < 8; ++e) x[e] = 0.f;
+        }
+        if (y) {
+            load8<T>(y + c * 8, v); load8<T>(post + c * 8, g);
+#pragma unroll
+            for (int e = 0; e < 8; ++e) x[e] += v[e] * inv1 * g[e];
+        }
+        if (inj) {
+            load8<T>(inj + c * 8, g);
+#pragma unroll
+            for (int e = 0; e < 8; ++e) x[e] += g[e];
+        }
+        store8<float>(rn.x_out + c * 8, x);
     }
 }
 

@@ -164,6 +164,9 @@ struct ResidualNormArgs {
     float mult, eps;
 };
 void launch_residual_norm(int dtype, const ResidualNormArgs& a, int rows, hipStream_t st);
+// one row: residual_norm and the linear that reads xn in ONE launch (a.X / a.norm_w come from rn; xn is never stored).  x_out must not be x_in
+bool gemv_residual_applies(int dtype, const GemvArgs& a);
+void launch_gemv_residual(int dtype, GemvArgs a, const ResidualNormArgs& rn, hipStream_t st);
 
 // rows of a prompt portion: q | k | v (| more) with head pitch D; per-head RMS norm over qk_dim (weights null = none), rotation of the first rot_dims dimensions (pairs
 // i, i + rot_dims / 2; table row = cos[rot_dims / 2] | sin[rot_dims / 2]), q back in place, k and v into the caches of launch_flash_prefill's layout

@@ -369,20 +369,34 @@ static WinDecodeArgs decode_args(const Stack& S, const StackLayer& l, const void
 void Model::stack_decode_step(Seq* s, hipStream_t st, int64_t* id_out) {
     Stack& S = *stk;
     const int dt = cfg.dtype;
-    float* xr = s->d_xr;
-    auto norm = [&](const float* xi, const void* yy, const StackStep& sp) {
-        LMX_PROF_K("decode.residual_norm");
-        launch_residual_norm(dt, ResidualNormArgs{xi, yy, sp.post, sp.inject ? s->d_h : nullptr, sp.pre, xr, s->d_x, H, S.c.width, S.c.residual_mult, S.c.norm_eps}, 1, st);
-    };
-    auto gemv = [&](const char* name, const void* xin, const void* w, void* c, const void* bias, int N, int K, int act) {
+    // the linear behind a norm: residual addition, both norms and the linear in one launch where the weight stream allows it (16-bit); the residual alternates between
+    // two rows because every workgroup of that launch reads the old one
+    float* xr[2] = {s->d_xr, s->d_xr + H};
+    int cur = -1;                                            // row that holds x (-1: none yet, x is the embedding row)
+    auto linear = [&](const char* name, const StackStep& sp, const void* y, GemvArgs g, bool fuse) {
+        const int nxt = cur == 0 ? 1 : 0;
+        const ResidualNormArgs rn{cur < 0 ? nullptr : xr[cur], y, sp.post, sp.inject ? s->d_h : nullptr, sp.pre, xr[nxt], s->d_x, H, S.c.width, S.c.residual_mult, S.c.norm_eps};
+        cur = nxt;
+        if (fuse && opt_stack_fuse && gemv_residual_applies(dt, g)) {
+            LMX_PROF_K(name);
+            launch_gemv_residual(dt, g, rn, st);
+            return;
+        }
+        { LMX_PROF_K("decode.residual_norm"); launch_residual_norm(dt, rn, 1, st); }
         LMX_PROF_K(name);
-        launch_gemv(dt, GemvArgs{xin, w, c, bias, nullptr, nullptr, 0.f, N, K, K, K, N, 0, act}, 1, st);
+        g.X = s->d_x;
+        launch_gemv(dt, g, 1, st);
     };
-    norm(nullptr, nullptr, StackStep{nullptr, S.layers[(size_t)S.runs[0].layer].n1, true});
+    auto plain = [&](const char* name, const void* xin, const void* w, void* c, int N, int K) {
+        LMX_PROF_K(name);
+        launch_gemv(dt, GemvArgs{xin, w, c, nullptr, nullptr, nullptr, 0.f, N, K, K, K, N, 0, kActNone}, 1, st);
+    };
+    StackStep before{nullptr, S.layers[(size_t)S.runs[0].layer].n1, true};
+    const void* y = nullptr;
     for (int r = 0; r < L; ++r) {
         const StackLayer& l = S.layers[(size_t)S.runs[(size_t)r].layer];
         const int an = l.c.n_heads * l.D;
-        gemv("decode.gemv.qkv", s->d_x, l.wqkv, s->d_qkv, l.bqkv, l.qkv_n, H, kActNone);
+        linear("decode.gemv.qkv", before, y, GemvArgs{nullptr, l.wqkv, s->d_qkv, l.bqkv, nullptr, nullptr, 0.f, l.qkv_n, H, H, H, l.qkv_n, 0, kActNone}, true);
         {
             LMX_PROF_K("decode.attn");
             WinDecodeArgs a = decode_args(S, l, s->d_qkv, s->d_attn, 1, s->len, s_max);
@@ -390,19 +404,18 @@ void Model::stack_decode_step(Seq* s, hipStream_t st, int64_t* id_out) {
             a.pos = s->len;
             launch_decode_win(dt, l.D, a, st);
         }
-        gemv("decode.gemv.o", s->d_attn, l.wo, s->d_y, nullptr, H, an, kActNone);
+        plain("decode.gemv.o", s->d_attn, l.wo, s->d_y, H, an);
+        y = s->d_y;
         if (l.ff) {
-            norm(xr, s->d_y, stack_step(S, r, 0, final_norm));
-            gemv("decode.gemv.gate_up", s->d_x, l.wgu, s->d_act, nullptr, 2 * l.ff, H, kActSiluMul);
-            gemv("decode.gemv.down", s->d_act, l.wd, s->d_y, nullptr, H, l.ff, kActNone);
+            linear("decode.gemv.gate_up", stack_step(S, r, 0, final_norm), y, GemvArgs{nullptr, l.wgu, s->d_act, nullptr, nullptr, nullptr, 0.f, 2 * l.ff, H, H, H, l.ff, 0, kActSiluMul}, true);
+            plain("decode.gemv.down", s->d_act, l.wd, s->d_y, H, l.ff);
         }
-        norm(xr, s->d_y, stack_step(S, r, l.ff ? 1 : 0, final_norm));
+        before = stack_step(S, r, l.ff ? 1 : 0, final_norm);
     }
     {
-        LMX_PROF_K("decode.gemv.lm_head");
-        GemvArgs ga{s->d_x, lm_head, s->d_logits, nullptr, nullptr, nullptr, 0.f, V, H, H, H, V, 0, kActNone};
+        GemvArgs ga{nullptr, lm_head, s->d_logits, nullptr, nullptr, nullptr, 0.f, V, H, H, H, V, 0, kActNone};
         ga.c_f32 = 1; ga.cap = S.c.logit_softcap;
-        launch_gemv(dt, ga, 1, st);
+        linear("decode.gemv.lm_head", before, y, ga, false);      // one row of residual_norm is cheaper than forming it in every workgroup of a vocabulary-wide linear
     }
     LMX_PROF("decode.argmax");
     const SeqStateRef ref{s->d_len, s->d_nout, s->d_tok, s->d_log, s->log_cap, 0, s->samp, s->d_stop};
