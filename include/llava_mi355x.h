@@ -332,6 +332,22 @@ size_t lmx_op_decode_attn_batch_tab_bytes(int32_t n_seq);
 size_t lmx_op_decode_attn_ws_bytes(int32_t n_rows, int32_t n_heads, int32_t n_split, int32_t head_dim);
 int lmx_op_sample(int32_t dtype, const void* logits_dev, int32_t V, float temperature, float top_p, int32_t top_k, uint64_t seed,
                   const int32_t* offset_dev, const uint32_t* u32_override_host, int64_t* out_tok_dev, uint8_t* keep_out_dev, void* stream);
+/* Kernels of the layer-stack decoders, one launch each (argument meaning: csrc/kernels.h ResidualNormArgs, QkvNormRopeArgs, FlashArgs' windowed form, WinDecodeArgs).
+ * linear_f32: fp32 output with soft cap; form 0 = GEMM, 1 = GEMV (M = 1), 2 = decode-batch kernel (M <= 32).  window_attn: rows_form 1 forces the vector-ALU kernel.
+ * decode_win: per-sequence pointers as lmx_op_decode_attn_batch (tab_dev: lmx_op_decode_attn_batch_tab_bytes(n_seq) bytes). */
+int lmx_op_residual_norm(int32_t dtype, const float* x_in, const void* y, const void* post_w, const void* inject, const void* pre_w, float* x_out, void* xn, int32_t rows,
+                         int32_t H, int32_t H_real, float mult, float eps, void* stream);
+int lmx_op_gemv_residual(int32_t dtype, const float* x_in, const void* y, const void* post_w, const void* inject, const void* pre_w, float* x_out, const void* w, const void* bias,
+                         void* c, int32_t N, int32_t H, int32_t H_real, float mult, float eps, int32_t act, void* stream);
+int lmx_op_linear_f32(int32_t dtype, const void* x, const void* w, float* c, int32_t M, int32_t N, int32_t K, float cap, int32_t form, void* stream);
+int lmx_op_qkv_norm_rope_kv(int32_t dtype, int32_t D, void* qkv, int32_t qkv_stride, void* kcache, void* vtcache, const void* q_norm, const void* k_norm, const float* cos_sin_dev,
+                            int32_t T, int32_t pos0, int32_t n_heads, int32_t n_kv_heads, int32_t s_max, int32_t qk_dim, int32_t rot_dims, float eps, void* stream);
+int lmx_op_window_attn(int32_t dtype, int32_t D, const void* q, int32_t q_stride, void* o, int32_t o_stride, const void* kcache, const void* vtcache, int32_t q_len, int32_t q_pos0,
+                       int32_t n_heads, int32_t n_kv_heads, int32_t s_max, float scale, int32_t window, int32_t sink, const void* gate, int32_t rows_form, void* stream);
+int lmx_op_decode_win(int32_t dtype, int32_t D, const void* qkv, int32_t qkv_stride, void* out, int32_t out_stride, void* const* kcaches, void* const* vtcaches,
+                      const int32_t* const* pos_devs, void* const* ws_devs, int32_t* const* counters_devs, int32_t n_seq, void* tab_dev, const void* q_norm, const void* k_norm,
+                      const float* cos_sin_dev, int32_t n_heads, int32_t n_kv_heads, int32_t s_max, int32_t n_split, int32_t qk_dim, int32_t rot_dims, int32_t window, int32_t sink,
+                      int32_t gate_off, float scale, float eps, void* stream);
 int lmx_op_argmax(int32_t dtype, const void* logits, int32_t V, int64_t* out_tok_dev, void* stream);
 int lmx_op_im2col(int32_t dtype, const void* pixels, void* out, int32_t N, int32_t S, int32_t patch, int32_t kpad, void* stream);
 

@@ -609,6 +609,67 @@ int lmx_op_im2col(int32_t dtype, const void* pixels, void* out, int32_t N, int32
     LMX_API_END
 }
 
+// ---- layer-stack decoders (stack_ops.hip) ----------------------------------------------------------------------------------------
+int lmx_op_residual_norm(int32_t dtype, const float* x_in, const void* y, const void* post_w, const void* inject, const void* pre_w, float* x_out, void* xn, int32_t rows,
+                         int32_t H, int32_t H_real, float mult, float eps, void* stream) {
+    LMX_API_BEGIN
+    launch_residual_norm(dtype, ResidualNormArgs{x_in, y, post_w, inject, pre_w, x_out, xn, H, H_real, mult, eps}, rows, S(stream));
+    LMX_API_END
+}
+int lmx_op_gemv_residual(int32_t dtype, const float* x_in, const void* y, const void* post_w, const void* inject, const void* pre_w, float* x_out, const void* w, const void* bias,
+                         void* c, int32_t N, int32_t H, int32_t H_real, float mult, float eps, int32_t act, void* stream) {
+    LMX_API_BEGIN
+    launch_gemv_residual(dtype, GemvArgs{nullptr, w, c, bias, nullptr, nullptr, 0.f, N, H, H, H, N, 0, act}, ResidualNormArgs{x_in, y, post_w, inject, pre_w, x_out, nullptr, H, H_real, mult, eps},
+                         S(stream));
+    LMX_API_END
+}
+int lmx_op_linear_f32(int32_t dtype, const void* x, const void* w, float* c, int32_t M, int32_t N, int32_t K, float cap, int32_t form, void* stream) {
+    LMX_API_BEGIN
+    LMX_REQUIRE(x && w && c && form >= 0 && form <= 2, "linear_f32: bad arguments");
+    if (form == 1) {
+        LMX_REQUIRE(M == 1, "linear_f32: the GEMV form has one row");
+        GemvArgs g{x, w, c, nullptr, nullptr, nullptr, 0.f, N, K, K, K, N, 0, kActNone};
+        g.c_f32 = 1; g.cap = cap;
+        launch_gemv(dtype, g, 1, S(stream));
+    } else {
+        GemmArgs g{x, w, c, nullptr, nullptr, M, N, K, K, K, N, 0, kActNone};
+        g.c_f32 = 1; g.cap = cap;
+        if (form == 2) launch_skinny_gemm(dtype, g, S(stream)); else launch_gemm(dtype, g, 0, S(stream));
+    }
+    LMX_API_END
+}
+int lmx_op_qkv_norm_rope_kv(int32_t dtype, int32_t D, void* qkv, int32_t qkv_stride, void* kcache, void* vtcache, const void* q_norm, const void* k_norm, const float* cos_sin_dev,
+                            int32_t T, int32_t pos0, int32_t n_heads, int32_t n_kv_heads, int32_t s_max, int32_t qk_dim, int32_t rot_dims, float eps, void* stream) {
+    LMX_API_BEGIN
+    launch_qkv_norm_rope_kv(dtype, D, QkvNormRopeArgs{qkv, kcache, vtcache, q_norm, k_norm, cos_sin_dev, T, pos0, qkv_stride, n_heads, n_kv_heads, s_max, qk_dim, rot_dims, eps}, S(stream));
+    LMX_API_END
+}
+int lmx_op_window_attn(int32_t dtype, int32_t D, const void* q, int32_t q_stride, void* o, int32_t o_stride, const void* kcache, const void* vtcache, int32_t q_len, int32_t q_pos0,
+                       int32_t n_heads, int32_t n_kv_heads, int32_t s_max, float scale, int32_t window, int32_t sink, const void* gate, int32_t rows_form, void* stream) {
+    LMX_API_BEGIN
+    FlashArgs a{q, o, kcache, vtcache, q_len, q_pos0 + q_len, q_pos0, q_stride, o_stride, n_heads, n_kv_heads, s_max, scale, 1};
+    a.win = 1; a.window = window; a.sink = sink; a.gate = gate;
+    if (rows_form || dtype == kF32 || D > 128) launch_rows_attn(dtype, D, a, S(stream)); else launch_flash_prefill(dtype, D, a, S(stream));
+    LMX_API_END
+}
+int lmx_op_decode_win(int32_t dtype, int32_t D, const void* qkv, int32_t qkv_stride, void* out, int32_t out_stride, void* const* kcaches, void* const* vtcaches,
+                      const int32_t* const* pos_devs, void* const* ws_devs, int32_t* const* counters_devs, int32_t n_seq, void* tab_dev, const void* q_norm, const void* k_norm,
+                      const float* cos_sin_dev, int32_t n_heads, int32_t n_kv_heads, int32_t s_max, int32_t n_split, int32_t qk_dim, int32_t rot_dims, int32_t window, int32_t sink,
+                      int32_t gate_off, float scale, float eps, void* stream) {
+    LMX_API_BEGIN
+    LMX_REQUIRE(n_seq >= 1 && kcaches && vtcaches && pos_devs && ws_devs && counters_devs && tab_dev, "decode_win: bad arguments");
+    std::vector<DecodeFusedSeq> tab((size_t)n_seq);
+    for (int i = 0; i < n_seq; ++i) tab[(size_t)i] = DecodeFusedSeq{kcaches[i], vtcaches[i], pos_devs[i], static_cast<float*>(ws_devs[i]), counters_devs[i]};
+    LMX_CHECK_HIP(hipMemcpyAsync(tab_dev, tab.data(), sizeof(DecodeFusedSeq) * (size_t)n_seq, hipMemcpyHostToDevice, S(stream)));
+    LMX_CHECK_HIP(hipStreamSynchronize(S(stream)));
+    WinDecodeArgs a;
+    a.qkv = qkv; a.out = out; a.q_norm = q_norm; a.k_norm = k_norm; a.cos_sin = cos_sin_dev; a.tab = static_cast<const DecodeFusedSeq*>(tab_dev);
+    a.n_seq = n_seq; a.qkv_stride = qkv_stride; a.out_stride = out_stride; a.n_heads = n_heads; a.n_kv_heads = n_kv_heads; a.s_max = s_max; a.n_split = n_split;
+    a.qk_dim = qk_dim; a.rot_dims = rot_dims; a.window = window; a.sink = sink; a.gate_off = gate_off; a.scale = scale; a.eps = eps;
+    launch_decode_win(dtype, D, a, S(stream));
+    LMX_API_END
+}
+
 // ---- training-step slices (train.hip) ---------------------------------------------------------------------------------------------
 int lmx_op_ce_loss(int32_t dtype, const void* logits, int32_t ld, const int64_t* labels, int32_t B, int32_t T, int32_t V, int64_t ignore_index,
                    float* lse_scratch, float* row_loss_scratch, float* out_loss_count, float grad, void* dlogits_or_null, int32_t ldd, void* stream) {

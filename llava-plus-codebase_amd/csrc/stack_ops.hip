@@ -101,10 +101,12 @@ void launch_residual_norm(int dtype, const ResidualNormArgs& a, int rows, hipStr
 }
 
 // ---------------------------------------------------------------------------------------------------------------
-// query / key norm + rotation + KV append of prompt rows.  grid (ceil(T / 64), H + 2 G), 256 threads: a group of D / 8 lanes owns one head vector, 8 consecutive
-// elements per lane; the rotation partner i +- dims / 2 comes through LDS (any even number of rotated dimensions).
+// query / key norm + rotation + KV append of prompt rows.  grid (ceil(T / 64), H + 2 G), 256 threads.
+//   PAIRED (rot_dims % 16 == 0): D / 16 lanes own one head vector, two 8-element chunks each — a chunk of the rotated part with its partner half a rotation away, or two
+//   neighbouring chunks of the rest — so a lane rotates what it loaded: no LDS, no barrier.
+//   otherwise: D / 8 lanes, 8 consecutive elements each, the partner i +- rot_dims / 2 through LDS (any even number of rotated dimensions).
 // ---------------------------------------------------------------------------------------------------------------
-template <typename T, int D>
+template <typename T, int D, bool PAIRED>
 __global__ __launch_bounds__(256) void qkv_norm_rope_kv_kernel(QkvNormRopeArgs a) {
     extern __shared__ __attribute__((aligned(16))) char smem[];
     const int tid = threadIdx.x;
@@ -112,6 +114,52 @@ __global__ __launch_bounds__(256) void qkv_norm_rope_kv_kernel(QkvNormRopeArgs a
     const int ntok = (a.T - tok0) < 64 ? (a.T - tok0) : 64;
     T* qkv = reinterpret_cast<T*>(a.qkv);
     constexpr int LPV = D / 8, VPP = 256 / LPV;          // lanes per vector, vectors per pass
+    if (PAIRED && slot < a.n_heads + a.n_kv_heads) {
+        constexpr int LP = D / 16, ITER = 64 * LP / 256;
+        const bool is_k = slot >= a.n_heads;
+        const int half8 = a.rot_dims >> 4, k = tid % LP;                   // rotated chunks per half
+        const bool rot = k < half8;
+        const int c0 = rot ? k : 2 * half8 + 2 * (k - half8), c1 = rot ? k + half8 : c0 + 1;
+        const T* nw = reinterpret_cast<const T*>(is_k ? a.k_norm : a.q_norm);
+        T* kc = reinterpret_cast<T*>(a.K) + (size_t)(is_k ? slot - a.n_heads : 0) * a.s_max * D;
+        float x[ITER][2][8], g0[8], g1[8];
+#pragma unroll
+        for (int it = 0; it < ITER; ++it) {
+            const int t = it * (256 / LP) + tid / LP;
+            const T* xp = qkv + (size_t)(tok0 + (t < ntok ? t : 0)) * a.qkv_stride + slot * D;
+            load8<T>(xp + c0 * 8, x[it][0]); load8<T>(xp + c1 * 8, x[it][1]);
+        }
+        if (nw) { load8<T>(nw + c0 * 8, g0); load8<T>(nw + c1 * 8, g1); }
+#pragma unroll
+        for (int it = 0; it < ITER; ++it) {
+            const int t = it * (256 / LP) + tid / LP;
+            const bool live = t < ntok;
+            float (&u)[8] = x[it][0];
+            float (&v)[8] = x[it][1];
+            if (nw) {
+                float ss = 0.f;
+#pragma unroll
+                for (int e = 0; e < 8; ++e) ss += u[e] * u[e] + v[e] * v[e];
+#pragma unroll
+                for (int o = LP / 2; o > 0; o >>= 1) ss += __shfl_xor(ss, o, 64);
+                const float inv = 1.f / sqrtf(ss / (float)a.qk_dim + a.eps);
+#pragma unroll
+                for (int e = 0; e < 8; ++e) { u[e] *= inv * g0[e]; v[e] *= inv * g1[e]; }
+            }
+            if (!live) continue;
+            const int pos = a.pos0 + tok0 + t;
+            if (rot) {
+                const float* cs = a.cos_sin + (size_t)pos * a.rot_dims + k * 8;
+                float c[8], s[8];
+                load8<float>(cs, c); load8<float>(cs + half8 * 8, s);
+#pragma unroll
+                for (int e = 0; e < 8; ++e) { const float p = u[e], q = v[e]; u[e] = p * c[e] - q * s[e]; v[e] = q * c[e] + p * s[e]; }
+            }
+            T* o = is_k ? kc + (size_t)pos * D : qkv + (size_t)(tok0 + t) * a.qkv_stride + slot * D;
+            store8<T>(o + c0 * 8, u); store8<T>(o + c1 * 8, v);
+        }
+        return;
+    }
     if (slot < a.n_heads + a.n_kv_heads) {
         float* vec = reinterpret_cast<float*>(smem);     // [VPP][D] normalised vectors of this pass
         const bool is_k = slot >= a.n_heads;
@@ -183,12 +231,13 @@ void launch_qkv_norm_rope_kv(int dtype, int D, const QkvNormRopeArgs& a, hipStre
     LMX_REQUIRE(a.pos0 >= 0 && a.pos0 + a.T <= a.s_max, "qkv_norm_rope_kv: rows past the cache");
     if (a.T <= 0) return;
     const dim3 grid(cdiv(a.T, 64), a.n_heads + 2 * a.n_kv_heads);
+    const bool paired = a.rot_dims % 16 == 0;
     size_t smem = (size_t)64 * (D + 2) * dtype_size(dtype);
-    if (smem < 256 * 8 * sizeof(float)) smem = 256 * 8 * sizeof(float);
+    if (!paired && smem < 256 * 8 * sizeof(float)) smem = 256 * 8 * sizeof(float);
 #define L(TT, DD) do {                                                                                                                   \
-        auto kern = qkv_norm_rope_kv_kernel<TT, DD>;                                                                                     \
-        static bool attr_set = false;                                                                                                    \
-        if (!attr_set) { LMX_CHECK_HIP(hipFuncSetAttribute(reinterpret_cast<const void*>(kern), hipFuncAttributeMaxDynamicSharedMemorySize, 80 * 1024)); attr_set = true; } \
+        auto kern = paired ? qkv_norm_rope_kv_kernel<TT, DD, true> : qkv_norm_rope_kv_kernel<TT, DD, false>;                                                                                     \
+        static bool attr_set[2] = {false, false};                                                                                        \
+        if (!attr_set[paired]) { LMX_CHECK_HIP(hipFuncSetAttribute(reinterpret_cast<const void*>(kern), hipFuncAttributeMaxDynamicSharedMemorySize, 80 * 1024)); attr_set[paired] = true; } \
         hipLaunchKernelGGL(kern, grid, dim3(256), smem, st, a);                                                                          \
     } while (0)
 #define LD(TT) do { if (D == 256) L(TT, 256); else if (D == 128) L(TT, 128); else L(TT, 64); } while (0)

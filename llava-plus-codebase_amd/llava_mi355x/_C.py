@@ -139,6 +139,12 @@ _SIGS = {
     "lmx_op_decode_attn_batch_tab_bytes": (c_size_t, [c_int32]),
     "lmx_op_decode_attn_ws_bytes": (c_size_t, [c_int32] * 4),
     "lmx_op_sample": (c_int32, [c_int32, c_void_p, c_int32, c_float, c_float, c_int32, ctypes.c_uint64, c_void_p, POINTER(ctypes.c_uint32), c_void_p, c_void_p, c_void_p]),
+    "lmx_op_residual_norm": (c_int32, [c_int32] + [c_void_p] * 7 + [c_int32] * 3 + [c_float, c_float, c_void_p]),
+    "lmx_op_gemv_residual": (c_int32, [c_int32] + [c_void_p] * 9 + [c_int32] * 3 + [c_float, c_float, c_int32, c_void_p]),
+    "lmx_op_linear_f32": (c_int32, [c_int32] + [c_void_p] * 3 + [c_int32] * 3 + [c_float, c_int32, c_void_p]),
+    "lmx_op_qkv_norm_rope_kv": (c_int32, [c_int32, c_int32, c_void_p, c_int32] + [c_void_p] * 5 + [c_int32] * 7 + [c_float, c_void_p]),
+    "lmx_op_window_attn": (c_int32, [c_int32, c_int32, c_void_p, c_int32, c_void_p, c_int32, c_void_p, c_void_p] + [c_int32] * 5 + [c_float, c_int32, c_int32, c_void_p, c_int32, c_void_p]),
+    "lmx_op_decode_win": (c_int32, [c_int32, c_int32, c_void_p, c_int32, c_void_p, c_int32] + [POINTER(c_void_p)] * 5 + [c_int32] + [c_void_p] * 4 + [c_int32] * 9 + [c_float, c_float, c_void_p]),
     "lmx_op_argmax": (c_int32, [c_int32, c_void_p, c_int32, c_void_p, c_void_p]),
     "lmx_op_ce_loss": (c_int32, [c_int32, c_void_p, c_int32, c_void_p, c_int32, c_int32, c_int32, c_int64, c_void_p, c_void_p, c_void_p, c_float, c_void_p, c_int32, c_void_p]),
     "lmx_op_rmsnorm_bwd": (c_int32, [c_int32, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int32, c_int32, c_float, c_void_p]),

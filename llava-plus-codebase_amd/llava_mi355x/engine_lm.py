@@ -219,6 +219,15 @@ class EngineCausalLM:
         if self._img_cache is not None:
             self._img_cache.clear()
 
+    def prefill_logits(self, caches: Sequence["LmxKVCache"], embeds: Sequence[torch.Tensor], wants: Sequence[Sequence[int]]) -> torch.Tensor:
+        """Continue several one-sequence caches by the rows in `embeds` ([T_i, row_pitch]) and return the logits of chosen rows, [sum len(wants[i]), _vocab_cap], in order
+        (`wants[i]`: ascending row indices of portion i).  A family whose engine serves that in one packed prefill overrides this."""
+        rows = []
+        for c, e, w in zip(caches, embeds, wants):
+            lg = self._prefill_rows(c, e[None], None, want_all=True, greedy=False)[0]
+            rows.append(lg[list(w)])
+        return torch.cat(rows)
+
     def _prefill_rows(self, cache: LmxKVCache, embeds: torch.Tensor, valid: Optional[torch.Tensor], want_all: bool, greedy: bool, chunk: int = 0):
         """Run the decoder over [B,T,H] embeddings; `valid` [B,T] bool marks real (non-pad) positions."""
         B, T, H = embeds.shape

@@ -194,6 +194,74 @@ def decode_kv_attn(q_row, x, w_kv, norm_w, eps, kcache, vtcache, cos_sin, pos, n
     return out
 
 
+# ---- layer-stack decoders (csrc/stack_ops.hip) ---------------------------------------------------------------------------------------------------
+def residual_norm(x_in, y, post_w, inject, pre_w, mult, eps, width=None, dtype=torch.bfloat16):
+    """x = x_in + mult rms_norm(y) post_w + inject; (x, rms_norm(x) pre_w).  x_in [rows, H] fp32 or None; the rest of `dtype` or None; means over `width` elements."""
+    _need_cuda(x_in, y, post_w, inject, pre_w)
+    ref = next(t for t in (x_in, y, inject) if t is not None)
+    rows, H = ref.shape
+    x = torch.empty((rows, H), dtype=torch.float32, device=ref.device)
+    xn = torch.empty((rows, H), dtype=dtype, device=ref.device) if pre_w is not None else None
+    check(lib.lmx_op_residual_norm(torch_dtype_code(dtype), ptr(x_in), ptr(y), ptr(post_w), ptr(inject), ptr(pre_w), ptr(x), ptr(xn), rows, H, width or H, mult, eps, stream_handle()),
+          "residual_norm")
+    return x, xn
+
+
+def gemv_residual(x_in, y, post_w, inject, pre_w, w, mult, eps, bias=None, width=None, act=_C.ACT_NONE):
+    """residual_norm of one row and the linear on its result in one launch: (x, act(xn @ w.T + bias))."""
+    _need_cuda(x_in, y, post_w, inject, pre_w, w, bias)
+    N, H = w.shape
+    x = torch.empty((1, H), dtype=torch.float32, device=w.device)
+    c = torch.empty((1, N // 2 if act == _C.ACT_SILU_MUL else N), dtype=w.dtype, device=w.device)
+    check(lib.lmx_op_gemv_residual(torch_dtype_code(w.dtype), ptr(x_in), ptr(y), ptr(post_w), ptr(inject), ptr(pre_w), ptr(x), ptr(w), ptr(bias), ptr(c), N, H, width or H, mult, eps, act,
+                                   stream_handle()), "gemv_residual")
+    return x, c
+
+
+def linear_f32(x, w, cap=0.0, form=0):
+    """x @ w.T with fp32 output, soft-capped; form 0 GEMM, 1 GEMV, 2 decode-batch kernel."""
+    _need_cuda(x, w)
+    out = torch.empty((x.shape[0], w.shape[0]), dtype=torch.float32, device=x.device)
+    check(lib.lmx_op_linear_f32(torch_dtype_code(x.dtype), ptr(x), ptr(w), ptr(out), x.shape[0], w.shape[0], x.shape[1], cap, form, stream_handle()), "linear_f32")
+    return out
+
+
+def qkv_norm_rope_kv(qkv, kcache, vtcache, q_norm, k_norm, cos_sin, pos0, n_heads, n_kv_heads, qk_dim, rot_dims, eps):
+    """Rows of a prompt portion: per-head norm, rotation, append; q in place.  Caches [G, s_max, D] / [G, D, s_max]."""
+    _need_cuda(qkv, kcache, vtcache, q_norm, k_norm, cos_sin)
+    D, s_max = kcache.shape[2], kcache.shape[1]
+    check(lib.lmx_op_qkv_norm_rope_kv(torch_dtype_code(qkv.dtype), D, ptr(qkv), qkv.stride(0), ptr(kcache), ptr(vtcache), ptr(q_norm), ptr(k_norm), ptr(cos_sin), qkv.shape[0], pos0,
+                                      n_heads, n_kv_heads, s_max, qk_dim, rot_dims, eps, stream_handle()), "qkv_norm_rope_kv")
+
+
+def window_attn(qkv, kcache, vtcache, q_pos0, n_heads, n_kv_heads, scale, window=0, sink=True, gate_off=-1, rows_form=False):
+    """Windowed causal attention of the rows of a prompt portion (rotated q heads in the first columns of qkv)."""
+    _need_cuda(qkv, kcache, vtcache)
+    D, s_max = kcache.shape[2], kcache.shape[1]
+    out = torch.empty((qkv.shape[0], n_heads * D), dtype=qkv.dtype, device=qkv.device)
+    gate = None if gate_off < 0 else qkv.data_ptr() + gate_off * qkv.element_size()
+    check(lib.lmx_op_window_attn(torch_dtype_code(qkv.dtype), D, ptr(qkv), qkv.stride(0), ptr(out), out.stride(0), ptr(kcache), ptr(vtcache), qkv.shape[0], q_pos0, n_heads, n_kv_heads,
+                                 s_max, scale, window, int(sink), gate, int(rows_form), stream_handle()), "window_attn")
+    return out
+
+
+def decode_win(qkv, kcaches, vtcaches, pos_words, cos_sin, n_heads, n_kv_heads, qk_dim, rot_dims, scale, eps, q_norm=None, k_norm=None, window=0, sink=True, gate_off=-1, n_split=1):
+    """One new token per sequence (row i of qkv, pre-norm, pre-rotation): append to cache i at its position word, windowed attention.  Returns [n_seq, n_heads * D]."""
+    import ctypes
+    _need_cuda(qkv, cos_sin, q_norm, k_norm, *kcaches, *vtcaches, *pos_words)
+    n = qkv.shape[0]
+    D, s_max = kcaches[0].shape[2], kcaches[0].shape[1]
+    out = torch.empty((n, n_heads * D), dtype=qkv.dtype, device=qkv.device)
+    ws = [torch.empty(n_heads * n_split * (D + 4), dtype=torch.float32, device=qkv.device) for _ in range(n)]
+    cnt = [torch.zeros(n_heads, dtype=torch.int32, device=qkv.device) for _ in range(n)]
+    tab = torch.empty(lib.lmx_op_decode_attn_batch_tab_bytes(n), dtype=torch.uint8, device=qkv.device)
+    arr = lambda ts: (ctypes.c_void_p * n)(*[t.data_ptr() for t in ts])
+    check(lib.lmx_op_decode_win(torch_dtype_code(qkv.dtype), D, ptr(qkv), qkv.stride(0), ptr(out), out.stride(0), arr(kcaches), arr(vtcaches), arr(pos_words), arr(ws), arr(cnt), n, ptr(tab),
+                                ptr(q_norm), ptr(k_norm), ptr(cos_sin), n_heads, n_kv_heads, s_max, n_split, qk_dim, rot_dims, window, int(sink), gate_off, scale, eps, stream_handle()),
+          "decode_win")
+    return out
+
+
 def argmax(logits):
     _need_cuda(logits)
     out = torch.zeros(1, dtype=torch.int64, device=logits.device)

@@ -159,6 +159,18 @@ class SiteraxForCausalLM(EngineCausalLM):
         l = self.config.layers
         return lib.lmx_layer_runs(self._h), max(x.kv_heads for x in l), max(x.dim for x in l)
 
+    def prefill_logits(self, caches, embeds, wants) -> torch.Tensor:
+        n, total = len(caches), sum(len(w) for w in wants)
+        logits = torch.empty((total, self._vocab_cap), dtype=torch.float32, device=self.device)
+        embeds = [e.to(self.dtype).contiguous() for e in embeds]
+        arr = (ctypes.c_void_p * n)(*[c.seqs[0].value for c in caches])
+        eptr = (ctypes.c_void_p * n)(*[e.data_ptr() for e in embeds])
+        cnt = (ctypes.c_int32 * n)(*[e.shape[0] for e in embeds])
+        nw = (ctypes.c_int32 * n)(*[len(w) for w in wants])
+        wr = (ctypes.c_int32 * max(1, total))(*[int(r) for w in wants for r in w])
+        check(lib.lmx_prefill_batch_logits(self._h, arr, n, eptr, cnt, 0, nw, wr, ptr(logits), 0, stream_handle()), "lmx_prefill_batch_logits")
+        return logits
+
     @torch.inference_mode()
     def forward(self, input_ids: torch.Tensor, past_key_values: Optional[LmxKVCache] = None, use_cache: bool = True, output_hidden_states: bool = False, chunk: int = 0,
                 **_unused) -> CausalLMOutput:

@@ -12,7 +12,6 @@ The family is chosen by config.json (registry.py); sequences, packed prefill, de
 from __future__ import annotations
 
 import argparse
-import ctypes
 import json
 import os
 import sys
@@ -20,7 +19,6 @@ from typing import Dict, List
 
 import torch
 
-from ._C import check, lib, ptr, stream_handle
 from .batching import DecodeBatch
 from .engine_lm import EngineCausalLM, LmxKVCache
 from .registry import load_model
@@ -66,26 +64,13 @@ class TraceReplay:
         return torch.stack([rows[(e["id"], w)] for e, w in order])[:, :V].float().cpu()
 
     def _prefill(self, entries: List[dict], rows: Dict[tuple, torch.Tensor]) -> None:
-        m, n = self.model, len(entries)
-        flat = torch.tensor([t for e in entries for t in e["tokens"]], dtype=torch.long)
-        embeds = m.get_model().embed_tokens(flat)
-        counts = [len(e["tokens"]) for e in entries]
-        parts = list(embeds.split(counts))
+        m = self.model
+        embeds = m.get_model().embed_tokens(torch.tensor([t for e in entries for t in e["tokens"]], dtype=torch.long))
+        parts = list(embeds.split([len(e["tokens"]) for e in entries]))
         wants = [sorted(set(e["want"])) for e in entries]
-        total = sum(len(w) for w in wants)
-        logits = torch.empty((max(1, total), m._vocab_cap), dtype=torch.float32, device=m.device)
-        arr = (ctypes.c_void_p * n)(*[self.live[e["id"]].seqs[0].value for e in entries])
-        eptr = (ctypes.c_void_p * n)(*[p.data_ptr() for p in parts])
-        cnt = (ctypes.c_int32 * n)(*counts)
-        nw = (ctypes.c_int32 * n)(*[len(w) for w in wants])
-        wr = (ctypes.c_int32 * max(1, total))(*[r for w in wants for r in w])
-        check(lib.lmx_prefill_batch_logits(m._h, arr, n, eptr, cnt, 0, nw, wr, ptr(logits), 0, stream_handle()), "lmx_prefill_batch_logits")
-        i = 0
-        for e, w in zip(entries, wants):
-            for r in w:
-                rows[(e["id"], r)] = logits[i]
-                i += 1
-        torch.cuda.current_stream(m.device).synchronize()      # embeds may go
+        logits = m.prefill_logits([self.live[e["id"]] for e in entries], parts, wants)
+        for row, key in zip(logits, [(e["id"], r) for e, w in zip(entries, wants) for r in w]):
+            rows[key] = row
 
     def _decode(self, entries: List[dict], rows: Dict[tuple, torch.Tensor]) -> None:
         m, n = self.model, len(entries)
