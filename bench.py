@@ -885,6 +885,12 @@ def _time_decoder(model, T, ctx, new_tokens, steps, warmup, batches=(8, 32)):
     prefill(T).close()
     check(lib.lmx_decode(model._h, c.seqs[0], -1, 8, None, 1, stream_handle()), "lmx_decode")
     prof = model.profile_read()
+    if "decode.kv_attn" in prof:        # the LLaMA step hides its attention under the k | v projection: its stand-alone launches, for the per-kernel comparison only
+        model.set_option("decode_splitq", 0)
+        model.profile(True)
+        check(lib.lmx_decode(model._h, c.seqs[0], -1, 8, None, 1, stream_handle()), "lmx_decode")
+        prof.update({k: v for k, v in model.profile_read().items() if k in ("decode.attn", "decode.gemv.qkv")})
+        model.set_option("decode_splitq", 1)
     model.profile(False)
     n = batches[-1]
     cs = [prefill(ctx // 2) for _ in range(n)]

@@ -150,6 +150,7 @@ void Model::stack_load_weight(const std::string& name, const void* src, int ndim
         const int nh = d.n_heads, nk = d.n_kv_heads;
         if (sub == "norm1") vec(l.n1, W, H);
         else if (sub == "norm1b") vec(l.n1b, W, H);
+        else if ((sub == "norm2" || sub == "norm2b") && !d.ff) return;       // norms of a feed-forward the layer does not have
         else if (sub == "norm2" && d.ff) vec(l.n2, W, H);
         else if (sub == "norm2b" && d.ff) vec(l.n2b, W, H);
         else if (sub == "mix.q") heads(0, nh, d.qk_dim);
