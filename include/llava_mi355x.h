@@ -22,10 +22,10 @@
 extern "C" {
 #endif
 
-#define LMX_ABI_VERSION 1
+#define LMX_ABI_VERSION 2
 
 enum { LMX_DTYPE_F32 = 0, LMX_DTYPE_BF16 = 1, LMX_DTYPE_F16 = 2 };
-enum { LMX_ACT_NONE = 0, LMX_ACT_QUICK_GELU = 1, LMX_ACT_GELU_ERF = 2, LMX_ACT_SILU_MUL = 3 };
+enum { LMX_ACT_NONE = 0, LMX_ACT_QUICK_GELU = 1, LMX_ACT_GELU_ERF = 2, LMX_ACT_SILU_MUL = 3, LMX_ACT_RELU_MUL = 4 };
 enum { LMX_PROJ_LINEAR = 0, LMX_PROJ_MLP_GELU = 1, LMX_PROJ_IDENTITY = 2 };
 enum { LMX_FEATURE_PATCH = 0, LMX_FEATURE_CLS_PATCH = 1 };
 
@@ -71,8 +71,15 @@ int lmx_create(const lmx_config* cfg, lmx_model** out);
 int lmx_destroy(lmx_model* m);
 
 /* Layer-stack decoders: models described layer by layer on the same sequences, batches, samplers and entry points (lmx_prefill*, lmx_decode*, lmx_seq_*, lmx_batch_*).
- * Per layer x <- x + m norm1b(attention(norm1 x)), x <- x + m norm2b(mlp(norm2 x)) with RMS norms, an fp32 residual stream and fp32, optionally soft-capped logits.
- * Layers [loop_start, loop_stop) run loop_times times in a row on the same weights (own caches per pass; the embedding row is added before each pass but the first). */
+ * Per layer x <- x + m norm1b(mixer(norm1 x)), x <- x + m norm2b(mlp(norm2 x)) with RMS norms, an fp32 residual stream and fp32, optionally soft-capped logits; or, with
+ * `parallel`, x <- x + m (mixer(h) + mlp(h)), h = norm1 x.  Layers [loop_start, loop_stop) run loop_times times in a row on the same weights (own caches per pass); before
+ * each pass but the first the embedding row is added, or, with loop_mix, before EVERY pass x <- W [x; embedding row] ("loop.in").
+ *
+ * Mixers.  ATTENTION: softmax attention with per-head query / key norms, rotation, window, sink and gates as the fields say.  LATENT: queries through a normalised latent
+ * of q_rank values, keys and values through one of kv_rank (what the cache holds), no positions, window.  DELTA: gated delta rule with a decay per head and key channel:
+ * n_heads value heads of v_dim on n_kv_heads query / key heads of qk_dim, causal convolutions of conv_taps inputs, decay and output-gate projections of inner size
+ * decay_rank / gate_rank; its state (fp32) lives with the sequence.  Feed-forward: gated, or `experts` of them of which a row uses `top_experts`. */
+enum { LMX_MIXER_ATTENTION = 0, LMX_MIXER_LATENT = 1, LMX_MIXER_DELTA = 2 };
 typedef struct lmx_layer_config {
     int32_t n_heads, n_kv_heads, qk_dim, v_dim;
     float attn_scale;            /* factor on q . k */
@@ -83,7 +90,13 @@ typedef struct lmx_layer_config {
     int32_t out_gate;            /* 1: head h's output times sigmoid(W_g x)[h] */
     int32_t rope_dims;           /* leading dimensions rotated, pairs (i, i + rope_dims / 2); 0 = none */
     int32_t rope_table;          /* index for lmx_stack_set_rope */
-    int32_t ff;                  /* SiLU-gated feed-forward width, 0 = no feed-forward */
+    int32_t ff;                  /* gated feed-forward width (of one expert where there are experts), 0 = no feed-forward */
+    int32_t mixer;               /* LMX_MIXER_* */
+    int32_t parallel;            /* 1: mixer and feed-forward both read norm1's output, no norms behind them */
+    int32_t ff_act;              /* LMX_ACT_SILU_MUL (or 0) | LMX_ACT_RELU_MUL */
+    int32_t experts, top_experts;      /* 0 = dense */
+    int32_t q_rank, kv_rank;     /* LATENT */
+    int32_t conv_taps, decay_rank, gate_rank;      /* DELTA */
     int32_t reserved[8];
 } lmx_layer_config;
 typedef struct lmx_stack_config {
@@ -92,6 +105,12 @@ typedef struct lmx_stack_config {
     int32_t loop_start, loop_stop, loop_times;
     float norm_eps, residual_mult, logit_softcap;      /* logit_softcap 0 = none */
     int32_t gemm_variant;
+    int32_t tied_head;           /* 1: logits from the embedding table */
+    int32_t loop_mix;            /* 1: every pass of the loop begins with x <- W [x; embedding row] */
+    /* > 0: the embedding row of a token gets row (previous token * mul_prev + token * mul_cur) mod buckets of a second table, row `buckets` for a sequence's first token.
+     * The engine then takes token ids as input rows (lmx_input_pitch elements wide: the id's bits), because a row depends on the token before it */
+    int32_t bigram_buckets;
+    int64_t bigram_mul_prev, bigram_mul_cur;
     int32_t reserved[8];
 } lmx_stack_config;
 int lmx_create_stack(const lmx_stack_config* cfg, const lmx_layer_config* layers, lmx_model** out);
@@ -99,6 +118,8 @@ int lmx_create_stack(const lmx_stack_config* cfg, const lmx_layer_config* layers
 int lmx_stack_set_rope(lmx_model* m, int32_t table, int32_t dims, const float* host_cos_sin, int32_t n_pos);
 /* widths of the rows this model exchanges: embedding / residual rows (elements), logit rows (elements), dtype of logits, layer runs (cache slots; rows of a residual trace) */
 int lmx_row_pitch(const lmx_model* m);
+int lmx_input_pitch(const lmx_model* m);      /* elements of an input row of lmx_prefill* (lmx_gather_embeds writes such rows): the embedding row, or the id (see bigram_buckets) */
+int lmx_recurrent(const lmx_model* m);        /* 1: a sequence carries state that cannot be cut back to an earlier position (lmx_seq_truncate keeps all of it or nothing) */
 int lmx_vocab_pitch(const lmx_model* m);
 int lmx_logit_dtype(const lmx_model* m);
 int lmx_layer_runs(const lmx_model* m);

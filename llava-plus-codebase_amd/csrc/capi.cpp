@@ -53,6 +53,8 @@ int lmx_stack_set_rope(lmx_model* m, int32_t table, int32_t dims, const float* h
     LMX_API_END
 }
 int lmx_row_pitch(const lmx_model* m) { return m ? m->impl.H : -1; }
+int lmx_input_pitch(const lmx_model* m) { return m ? m->impl.input_pitch() : -1; }
+int lmx_recurrent(const lmx_model* m) { return m ? (m->impl.fixed_context() ? 1 : 0) : -1; }
 int lmx_vocab_pitch(const lmx_model* m) { return m ? m->impl.V : -1; }
 int lmx_logit_dtype(const lmx_model* m) { return m ? m->impl.logit_dtype() : -1; }
 int lmx_layer_runs(const lmx_model* m) { return m ? m->impl.L : -1; }
@@ -209,7 +211,7 @@ int lmx_seq_create(lmx_model* m, lmx_seq** out) {
         std::lock_guard<std::mutex> lk(m->impl.pool_mu);
         if (!m->impl.seq_pool.empty()) {
             s = m->impl.seq_pool.back(); m->impl.seq_pool.pop_back();
-            m->impl.seq_pool_bytes -= s->impl.kc.bytes + s->impl.vt.bytes + s->impl.dws.bytes + s->impl.pws.bytes;
+            m->impl.seq_pool_bytes -= s->impl.pool_bytes();
         }
     }
     if (s) {
@@ -248,7 +250,7 @@ int lmx_seq_destroy(lmx_seq* s) {
     if (m && idle_known && s->impl.pws.bytes > kPwsKeepMax) { s->impl.pws.release(); s->impl.pws_tokens = 0; }
     if (m && idle_known) {
         std::lock_guard<std::mutex> lk(m->pool_mu);
-        const size_t bytes = s->impl.kc.bytes + s->impl.vt.bytes + s->impl.dws.bytes + s->impl.pws.bytes;
+        const size_t bytes = s->impl.pool_bytes();
         if (m->seq_pool.size() < m->seq_pool_max && m->seq_pool_bytes + bytes <= m->seq_pool_bytes_max) {
             m->seq_pool.push_back(s); m->seq_pool_bytes += bytes; pooled = true;
         }
@@ -807,6 +809,7 @@ int lmx_seq_truncate(lmx_seq* s, int32_t n_rows, void* stream) {
     LMX_API_BEGIN
     LMX_REQUIRE(s, "null sequence");
     LMX_REQUIRE(n_rows >= 0 && n_rows <= s->impl.len, "seq_truncate: 0 <= n_rows <= current length");
+    LMX_REQUIRE(n_rows == 0 || n_rows == s->impl.len || !s->impl.m->fixed_context(), "seq_truncate: this model's sequences carry state that cannot be cut back");
     // a finished request's sequence starts another request that shares its first n_rows positions (prefix reuse): keep K / V^T rows [0, n_rows), forget the
     // rest of the request — position, token log, sampling parameters, stop rule (ordered on `stream` behind whatever still runs on the sequence)
     s->impl.len = n_rows;

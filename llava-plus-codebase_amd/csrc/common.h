@@ -161,11 +161,14 @@ template <int NW> __device__ __forceinline__ float block_max(float v, float* red
 }
 
 // ---- activations (epilogue codes; mirrors include/llava_mi355x.h LMX_ACT_*) -------------------
-enum Act : int { kActNone = 0, kActQuickGelu = 1, kActGeluErf = 2, kActSiluMul = 3 };
+enum Act : int { kActNone = 0, kActQuickGelu = 1, kActGeluErf = 2, kActSiluMul = 3, kActReluMul = 4 };
+// gated forms: the weight's rows come in [32 gate | 32 up] groups and the output is f(gate) * up
+__host__ __device__ __forceinline__ bool act_gated(int act) { return act == kActSiluMul || act == kActReluMul; }
 
 __device__ __forceinline__ float act_quick_gelu(float x) { return x / (1.f + __expf(-1.702f * x)); }
 __device__ __forceinline__ float act_gelu_erf(float x) { return 0.5f * x * (1.f + erff(x * 0.70710678118654752f)); }
 __device__ __forceinline__ float act_silu(float x) { return x / (1.f + __expf(-x)); }
+__device__ __forceinline__ float gate_mul(int act, float g, float u) { return (act == kActReluMul ? fmaxf(g, 0.f) : act_silu(g)) * u; }
 
 // logits <- cap tanh(logits / cap); cap <= 0: unchanged
 __device__ __forceinline__ float soft_cap(float v, float cap) { return cap > 0.f ? cap * tanhf(v / cap) : v; }

@@ -526,6 +526,14 @@ void launch_set_state(int* len_ptr, int len, int64_t* tok_ptr, int64_t tok, int 
 }
 
 
+__global__ void set_prev_kernel(int64_t* prev, const int* id, const int64_t* from) {
+    if (threadIdx.x == 0 && blockIdx.x == 0) *prev = id ? (int64_t)*id : *from;
+}
+void launch_set_prev(int64_t* prev, const int* id, const int64_t* from, hipStream_t st) {
+    hipLaunchKernelGGL(set_prev_kernel, dim3(1), dim3(64), 0, st, prev, id, from);
+    LMX_CHECK_HIP(hipGetLastError());
+}
+
 // 128-bit content hash of a device buffer (image-feature cache key: the LLaVA-Plus tool loop re-sends the same image with every re-prompt,
 // llava/serve/gradio_web_server_llava_plus.py:612-637).  Two independent 64-bit sums of mixed 16-byte chunks: each chunk is mixed with its index, the sums are
 // commutative (atomic adds in any order give the same value), so the hash is a pure function of the bytes.  n16 = number of 16-byte chunks; `tail` bytes (< 16)

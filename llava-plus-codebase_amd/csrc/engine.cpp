@@ -508,6 +508,10 @@ void Model::encode_images(const void* pixels, int n, void* feats, hipStream_t st
 
 void Model::gather_embeds(const int32_t* src, int rows, const void* feats, void* out, hipStream_t st) {
     LMX_REQUIRE(embed != nullptr, "embed_tokens not loaded");
+    if (stk && stk->ids_in()) {          // input rows of this model are the ids themselves
+        LMX_CHECK_HIP(hipMemcpyAsync(out, src, (size_t)rows * sizeof(int32_t), hipMemcpyDeviceToDevice, st));
+        return;
+    }
     launch_gather_embed(cfg.dtype, src, embed, feats, out, rows, H, st);
 }
 
@@ -521,14 +525,14 @@ uint64_t next_seq_uid() { return g_seq_uid.fetch_add(1); }
 Seq::Seq(Model* mm) : m(mm) {
     uid = g_seq_uid.fetch_add(1);
     layer_stride = (size_t)m->nkv_l * m->s_max * m->D * m->es;
-    const size_t kv_bytes = m->stk ? m->stk->kv_bytes : layer_stride * m->L;
-    kc.ensure(kv_bytes, true);
-    vt.ensure(kv_bytes, true);
+    if (m->stk) { if (m->stk->k_bytes) kc.ensure(m->stk->k_bytes, true); if (m->stk->v_bytes) vt.ensure(m->stk->v_bytes, true); if (m->stk->s_bytes) rs.ensure(m->stk->s_bytes, true); }
+    else { kc.ensure(layer_stride * m->L, true); vt.ensure(layer_stride * m->L, true); }
     log_cap = m->s_max + 8;
-    state.ensure(16 + (size_t)log_cap * 8, true);
+    state.ensure(16 + (size_t)log_cap * 8 + 8, true);
     d_len = state.as<int>(); d_nout = d_len + 1;
     d_tok = reinterpret_cast<int64_t*>(state.as<char>() + 8);
     d_log = d_tok + 1;
+    d_prev = d_log + log_cap;
     stopbuf.ensure(sizeof(StopSpec), true);
     d_stop = stopbuf.as<StopSpec>();
     // decode workspace
@@ -537,15 +541,16 @@ Seq::Seq(Model* mm) : m(mm) {
     const size_t aws = m->stk ? m->stk->dec_ws : decode_fused_ws_floats(m->nh_l, n_split, m->D);
     size_t off = 0;
     auto carve = [&](size_t bytes) { size_t o = off; off += (bytes + 255) / 256 * 256; return o; };
-    const size_t o_h = carve((size_t)m->H * es), o_qkv = carve((size_t)m->qkv_n * es), o_attn = carve((size_t)m->nh_l * m->D * es),
+    const size_t o_h = carve((size_t)m->H * es), o_qkv = carve((size_t)m->qkv_n * es), o_attn = carve((size_t)(m->stk ? m->stk->mix_n : m->nh_l * m->D) * es),
                  o_act = carve((size_t)m->I_l * es), o_log = carve((size_t)m->V * m->les), o_aws = carve(aws * 4), o_cnt = carve((size_t)m->nh_l * 4);
     const size_t o_x = m->stk ? carve((size_t)m->H * es) : 0, o_y = m->stk ? carve((size_t)m->H * es) : 0, o_xr = m->stk ? carve((size_t)m->H * 8) : 0;
+    const size_t o_sw = m->stk ? carve(m->stk->ws_bytes(1, m->H, es, true)) : 0;
     dws.ensure(off, true);
     char* W = dws.as<char>();
     d_h = W + o_h; d_qkv = W + o_qkv; d_attn = W + o_attn; d_act = W + o_act; d_logits = W + o_log;
     d_aws = reinterpret_cast<float*>(W + o_aws);
     d_cnt = reinterpret_cast<int*>(W + o_cnt);
-    if (m->stk) { d_x = W + o_x; d_y = W + o_y; d_xr = reinterpret_cast<float*>(W + o_xr); }
+    if (m->stk) { d_x = W + o_x; d_y = W + o_y; d_xr = reinterpret_cast<float*>(W + o_xr); sw = m->stk->ws(W + o_sw, 1, m->H, es, true); }
     kv_gran.ensure((size_t)2 * m->nkv_l * m->D * 8, true);
     LMX_CHECK_HIP(hipHostMalloc(reinterpret_cast<void**>(&h_status), sizeof(unsigned), hipHostMallocMapped));
     *h_status = 0;
@@ -912,7 +917,7 @@ void Model::decode(Seq* s, int64_t token, int n_steps, void* logits, bool greedy
     // Plain stream launches: the ~160 kernels of a step average >20 us each against ~3.5 us of host launch cost, so the
     // host runs far ahead of the GPU; a captured hipGraph measured no faster (3.57 vs 3.56 ms/token, profiles/EXPERIMENTS.md)
     // and stream capture is not safe next to other threads using the legacy stream (model_worker runs 5 request threads).
-    { LMX_PROF("decode.embed"); launch_gather_token(cfg.dtype, s->d_tok, embed, s->d_h, H, V, st); }
+    if (!stk || !stk->ids_in()) { LMX_PROF("decode.embed"); launch_gather_token(cfg.dtype, s->d_tok, embed, s->d_h, H, V, st); }      // (otherwise every step begins with its own row)
     for (int i = 0; i < n_steps; ++i) {
         decode_step_launch(s, st);
         s->len += 1;
@@ -956,16 +961,17 @@ Batch::Batch(Model* mm, int capacity) : m(mm), cap(capacity) {
     size_t off = 0;
     auto carve = [&](size_t bytes) { size_t o = off; off += (bytes + 255) / 256 * 256; return o; };
     const size_t o_h = carve((size_t)cap * m->H * es), o_x = carve((size_t)cap * m->H * es), o_qkv = carve((size_t)cap * m->qkv_n * es),
-                 o_attn = carve((size_t)cap * m->nh_l * m->D * es), o_act = carve((size_t)cap * m->I_l * es), o_log = carve((size_t)cap * m->V * m->les);
+                 o_attn = carve((size_t)cap * (m->stk ? m->stk->mix_n : m->nh_l * m->D) * es), o_act = carve((size_t)cap * m->I_l * es), o_log = carve((size_t)cap * m->V * m->les);
     const size_t o_y = m->stk ? carve((size_t)cap * m->H * es) : 0, o_xr = m->stk ? carve((size_t)cap * m->H * 4) : 0;
+    const size_t o_sw = m->stk ? carve(m->stk->ws_bytes(cap, m->H, es, true)) : 0;
     ws.ensure(off, true);
     char* W = ws.as<char>();
     h = W + o_h; x = W + o_x; qkv = W + o_qkv; attn = W + o_attn; act = W + o_act; logits = W + o_log;
-    if (m->stk) { y = W + o_y; xr = reinterpret_cast<float*>(W + o_xr); }
+    if (m->stk) { y = W + o_y; xr = reinterpret_cast<float*>(W + o_xr); sw = m->stk->ws(W + o_sw, cap, m->H, es, true); }
     const size_t attn_bytes = sizeof(DecodeFusedSeq) * (size_t)m->L * cap, state_bytes = sizeof(SeqStateRef) * (size_t)cap;
     tab.ensure(attn_bytes + state_bytes, true);
     if (m->cfg.dtype != kF32) {                     // K-sliced linears of a decode batch: o_proj / down_proj (N = H) and q|k|v
-        const int nmax = std::max(m->H, m->qkv_n);
+        const int nmax = std::max(std::max(m->H, m->qkv_n), m->stk ? m->stk->q_n : 0);
         sk_scratch.ensure(skinny_scratch_bytes(nmax)); sk_cnt.ensure((size_t)(nmax / 64 + 1) * sizeof(int), true);
     }
     d_attn_tab = tab.as<DecodeFusedSeq>();
@@ -984,10 +990,10 @@ void Batch::bind(Seq* const* seqs, int n, hipStream_t st) {
     for (int i = 0; i < n; ++i) {
         Seq* s = seqs[i];
         for (int l = 0; l < L; ++l) {
-            const size_t off = m->stk ? m->stk->runs[(size_t)l].kv_off : (size_t)l * s->layer_stride;
-            at[(size_t)l * cap + i] = DecodeFusedSeq{s->kc.as<char>() + off, s->vt.as<char>() + off, s->d_len, s->d_aws, s->d_cnt};
+            const size_t off = (size_t)l * s->layer_stride;
+            at[(size_t)l * cap + i] = m->stk ? m->stack_seq_ref(l, s) : DecodeFusedSeq{s->kc.as<char>() + off, s->vt.as<char>() + off, s->d_len, s->d_aws, s->d_cnt};
         }
-        stt[i] = SeqStateRef{s->d_len, s->d_nout, s->d_tok, s->d_log, s->log_cap, 0, s->samp, s->d_stop};
+        stt[i] = SeqStateRef{s->d_len, s->d_nout, s->d_tok, s->d_log, s->log_cap, 0, s->samp, s->d_stop, m->stk && m->stk->ids_in() ? s->d_prev : nullptr};
     }
     // the previous step's kernels may still be reading the old tables on this stream, and the host image is reused
     LMX_CHECK_HIP(hipStreamSynchronize(st));
@@ -1038,14 +1044,14 @@ void Model::decode_batch(Batch* b, Seq* const* seqs, int n, const int64_t* token
     if (n == 1) {
         // a lone member takes the single-sequence step (GEMV with fused RMSNorm: fewer launches, full-rate weight stream)
         Seq* s = seqs[0];
-        launch_gather_token(dt, s->d_tok, embed, s->d_h, H, V, st);
+        if (!stk || !stk->ids_in()) launch_gather_token(dt, s->d_tok, embed, s->d_h, H, V, st);
         for (int step = 0; step < n_steps; ++step) {
             decode_step_launch(s, st, d_ids + (size_t)step * b->cap);      // a lone member reports -1 after a device-side stop exactly like the members of a larger batch
             s->len += 1;
         }
         if (logits) LMX_CHECK_HIP(hipMemcpyAsync(logits, s->d_logits, (size_t)V * les, hipMemcpyDeviceToDevice, st));
     } else {
-    { LMX_PROF("decode_batch.embed"); launch_gather_tokens_batch(dt, b->d_state_tab, n, embed, b->h, H, V, st); }
+    if (!stk || !stk->ids_in()) { LMX_PROF("decode_batch.embed"); launch_gather_tokens_batch(dt, b->d_state_tab, n, embed, b->h, H, V, st); }
     for (int step = 0; step < n_steps; ++step) {
         if (stk) {
             stack_decode_batch_step(b, seqs, n, d_ids + (size_t)step * b->cap, st);

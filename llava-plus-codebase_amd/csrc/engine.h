@@ -53,17 +53,36 @@ struct VisLayerW {
 // ---- layer-stack decoders (stack.cpp) ---------------------------------------------------------------------------------------------------------------------
 struct StackLayer {
     lmx_layer_config c{};
-    int D = 0, qkv_n = 0, ff = 0, gate_off = -1;         // padded head width, rows of the fused q | k | v | gate weight, padded ff (0: none), first gate row (-1: none)
+    int D = 0, qkv_n = 0, ff = 0, gate_off = -1;         // padded head width, rows of the fused projection (q | k | v | gates), padded ff (0: none), first gate row (-1: none)
+    int an = 0, out_k = 0;                               // width of the mixer's output row; input width of `wo` (a parallel layer's dense down projection sits behind it: one product)
+    DeltaShape ds; int ra = 0, rg = 0;                   // delta: head shape, padded inner widths; projection rows q | k | v | beta | decay latent | gate latent
+    int a_off() const { return ds.channels() + (ds.H + 63) / 64 * 64; }
+    int Q = 0, R = 0;                                    // latent: padded widths; projection rows query latent | key / value latent
+    bool parallel() const { return c.parallel != 0; }
+    bool dense() const { return ff > 0 && c.experts == 0; }
+    bool moe() const { return ff > 0 && c.experts > 0; }
+    int act() const { return c.ff_act == LMX_ACT_RELU_MUL ? kActReluMul : kActSiluMul; }
+    void *conv = nullptr, *a_log = nullptr, *dt_bias = nullptr, *onorm = nullptr, *wag = nullptr;      // delta (wag: decay rows | gate rows over decay latent | gate latent)
+    void *qn_lat = nullptr, *kn_lat = nullptr, *wuq = nullptr, *wukv = nullptr, *wuk_t = nullptr;      // latent (wukv: [key rows | value rows] per head blocks of D; wuk_t [head][R][D])
+    void *wr = nullptr, *br = nullptr, *sw_uq = nullptr;                                               // router; wgu / wd hold all experts one after the other
     void *wqkv = nullptr, *bqkv = nullptr, *wo = nullptr, *wgu = nullptr, *wd = nullptr, *n1 = nullptr, *n1b = nullptr, *n2 = nullptr, *n2b = nullptr, *qn = nullptr, *kn = nullptr;
     void *sw_qkv = nullptr, *sw_o = nullptr, *sw_gu = nullptr, *sw_d = nullptr;
 };
-struct StackRun { int layer; bool inject; size_t kv_off; };      // one execution of a layer: own slice of the K and V^T caches (byte offset, same in both)
+// one execution of a layer: own slice of the K and V^T caches (byte offsets; a latent layer's rows are in the K cache) and of the recurrent state (state, ring).
+// inject: the embedding row is added first; mix: a pass of the loop begins (x <- W [x; embedding row])
+struct StackRun { int layer; bool inject, mix; size_t k_off, v_off, s_off, r_off; };
+struct StackWs { void *q, *qlat, *olat, *act, *slots, *cat; int* ids; float* wt; };      // activations beside the ones every decoder has
 struct Stack {
     lmx_stack_config c{};
     std::vector<StackLayer> layers;
     std::vector<StackRun> runs;
-    size_t kv_bytes = 0, dec_ws = 0;                     // bytes of one sequence's K (= V^T) cache; floats of its decode partials
-    int attn_n = 0;                                      // widest concatenation of heads
+    size_t k_bytes = 0, v_bytes = 0, s_bytes = 0, dec_ws = 0;      // bytes of one sequence's K and V^T caches and recurrent state; floats of its decode partials
+    int mix_n = 0;                                       // widest input row of an output projection
+    int q_n = 0, lat_n = 0, moe_act = 0, moe_top = 0;    // widest latent-attention query row, latent query row, expert activations and choices of a row
+    void *bigram = nullptr, *loop_in = nullptr, *sw_loop = nullptr;
+    bool ids_in() const { return c.bigram_buckets > 0; }
+    size_t ws_bytes(int rows, int H, int es, bool decode) const;
+    StackWs ws(void* base, int rows, int H, int es, bool decode) const;
     std::vector<float*> rope; std::vector<int> rope_dims;
     ~Stack() { for (float* p : rope) if (p) (void)hipFree(p); }
 };
@@ -143,6 +162,8 @@ struct Model {
 
     explicit Model(const lmx_config& c);
     Model(const lmx_stack_config& c, const lmx_layer_config* layers);
+    int input_pitch() const { return stk && stk->ids_in() ? 4 / es : H; }
+    bool fixed_context() const { return stk && (stk->s_bytes > 0 || stk->ids_in()); }
     int logit_dtype() const { return les == 4 ? (int)kF32 : cfg.dtype; }
     ~Model();
     void* alloc_weight(size_t bytes, bool zero = false);
@@ -177,7 +198,17 @@ struct Model {
     void stack_prefill(Seq* const* seqs, const void* const* embeds, const int* Ts, int n, int block_rows, bool greedy, const StackOutputs& out, hipStream_t st);
     void stack_decode_step(Seq* s, hipStream_t st, int64_t* id_out);
     void stack_decode_batch_step(struct Batch* b, Seq* const* seqs, int n, int64_t* ids, hipStream_t st);
+    DecodeFusedSeq stack_seq_ref(int r, Seq* s) const;      // what the kernels of run r need of a sequence
+    void stack_batch_linear(Batch* b, GemmArgs g, const void* wsw, hipStream_t st);
     void stack_seq_copy(Seq* dst, const Seq* src, hipStream_t st);
+    struct Segment { int seq, src0, dst0, n, pos0; };    // rows [src0, src0 + n) of sequence `seq` sit at rows [dst0, ...) of the piece; first position pos0
+    // a mixer over the normed rows x of a piece -> rows [an] of pitch out_k; qkv: its projection rows
+    void stack_mix_prefill(int r, Seq* const* seqs, const std::vector<Segment>& seg, int fill, const void* x, void* qkv, void* mix, void* scratch, void* skw, hipStream_t st);
+    size_t stack_mix_scratch(int rows, int keys) const;
+    void stack_moe_prefill(const StackLayer& l, const void* x, int rows, const StackWs& w, hipStream_t st);
+    // the same over one new token of every sequence (tab: batch; else `one`), projection rows already there
+    void stack_mix_decode(int r, const DecodeFusedSeq* tab, const DecodeFusedSeq& one, int n, int max_len, void* qkv, void* mix, const StackWs& w, Batch* b, hipStream_t st);
+    void stack_moe_decode(const StackLayer& l, const void* x, int n, const StackWs& w, bool batch, hipStream_t st);
     // ---- options a caller may flip on a live model (lmx_model_set_option; defaults from the environment at creation) ----------------------------------
     // fuse_rope: RoPE + KV append in the prefill's q|k|v GEMM epilogue (gemm8p.hip qkv_rope_epilogue) instead of a rope_kv launch — bit-identical, faster
     // vis_pack:  CLIP K / V^T pack in the tower's q|k|v GEMM epilogue instead of a pack launch — bit-identical, launch count
@@ -209,11 +240,14 @@ struct Seq {
     hipEvent_t ev_idle = nullptr;
     SampleParams samp;          // temperature <= 0: greedy; set by lmx_seq_set_sampling (bumps uid so a Batch re-reads it)
     DevBuf kc, vt;              // [L][nkv_l][s_max][D] and [L][nkv_l][D][s_max]
+    DevBuf rs;                  // recurrent state of a layer-stack decoder (per run: delta states and convolution rings); nothing of it is read at position 0
+    size_t pool_bytes() const { return kc.bytes + vt.bytes + rs.bytes + dws.bytes + pws.bytes; }
     size_t layer_stride = 0;    // bytes per layer in each cache
     int len = 0;                // host mirror of *d_len.  A device-side stop freezes *d_len while steps queued ahead still count here: resync_len()
     void resync_len(int dev_len, int dev_done) { if (dev_done != 0 && dev_len >= 0 && dev_len < len) len = dev_len; }   // called wherever the host has just read both
     DevBuf state;               // device: [0] int len, [1] int n_out, then int64 tok at byte 8, token log from byte 16
-    int* d_len = nullptr; int* d_nout = nullptr; int64_t* d_tok = nullptr; int64_t* d_log = nullptr;
+    int* d_len = nullptr; int* d_nout = nullptr; int64_t* d_tok = nullptr; int64_t* d_log = nullptr; int64_t* d_prev = nullptr;      // d_prev: the last token of the context (models whose embedding looks back)
+    StackWs sw{};
     DevBuf stopbuf; StopSpec* d_stop = nullptr;          // device-side stop rule (lmx_seq_set_stop); all zero = no rule
     int log_cap = 0;
     DevBuf pws;  int pws_tokens = 0;   // prefill workspace
@@ -242,9 +276,10 @@ struct Batch {
     int cap = 0;
     DevBuf ws;                         // h | x (normed) | qkv | attn | act | logits, each [cap][...]
     void *h = nullptr, *x = nullptr, *qkv = nullptr, *attn = nullptr, *act = nullptr, *logits = nullptr;
+    StackWs sw{};
     void* y = nullptr; float* xr = nullptr;      // layer-stack decoders: sublayer outputs, fp32 residual rows
     DevBuf tab;                        // device: DecodeFusedSeq[L][cap] then SeqStateRef[cap]
-    DecodeFusedSeq* d_attn_tab = nullptr; SeqStateRef* d_state_tab = nullptr;
+    DecodeFusedSeq* d_attn_tab = nullptr; SeqStateRef* d_state_tab = nullptr;      // [L][cap] (recurrent runs: K = state, VT = ring) and [cap]
     std::vector<uint64_t> members;     // Seq::uid of what the device tables currently describe
     std::vector<char> host_tab;
     DevBuf ids; int ids_steps = 0;     // [ids_steps][cap] int64: greedy picks of the chained steps of the last call
@@ -296,6 +331,7 @@ int splice_plan(const int64_t* input_ids, const uint8_t* attention_mask, const i
 
 // elementwise.hip (state helpers)
 void launch_set_state(int* len_ptr, int len, int64_t* tok_ptr, int64_t tok, int set_tok, int* nout_ptr, int set_nout, hipStream_t st);
+void launch_set_prev(int64_t* prev, const int* id, const int64_t* from, hipStream_t st);      // *prev = *id, or *from without an id
 void launch_set_stop(StopSpec* dst, const StopSpec& v, hipStream_t st);
 void launch_hash128(const void* base, size_t bytes_per_item, int items, uint64_t* out_dev, hipStream_t st);      // out_dev[2 * item + {0, 1}]      // *dst = v on the stream (v travels as a kernel argument; re-arms done = v.done)
 void launch_interleave_half(int dtype, const void* src, void* dst, int I, int K, int half, hipStream_t st);

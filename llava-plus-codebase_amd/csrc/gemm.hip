@@ -388,7 +388,7 @@ __global__ __launch_bounds__(256) void gemm_f32_kernel(GemmArgs a) {
             if (n >= a.N) continue;
             float v = acc[i][j];
             if (bias) v += bias[n];
-            if (act == kActSiluMul) {
+            if (act_gated(act)) {
                 // [32 gate | 32 up] interleave: this thread holds gate when (n % 64) < 32; its partner column n+32
                 // lives in thread tx+8 of the same row -> exchange through LDS is avoided by recomputing ownership:
                 // handled below by a second pass (see after loop)
@@ -401,7 +401,7 @@ __global__ __launch_bounds__(256) void gemm_f32_kernel(GemmArgs a) {
             C[(size_t)m * a.ldc + n] = v;
         }
     }
-    if (act == kActSiluMul) {
+    if (act_gated(act)) {
         // exchange through LDS: write the biased 64x64 tile, then gate threads combine with up values.
         __shared__ float Ts[64][64 + 1];
         __syncthreads();
@@ -420,7 +420,7 @@ __global__ __launch_bounds__(256) void gemm_f32_kernel(GemmArgs a) {
                     const int nl = tx * 4 + j;          // 0..31 gate column inside this 64 group
                     if (n0 + nl >= a.N) continue;
                     const float g = Ts[ty * 4 + i][nl], u = Ts[ty * 4 + i][nl + 32];
-                    C[(size_t)m * a.ldc + n0 / 2 + nl] = act_silu(g) * u;
+                    C[(size_t)m * a.ldc + n0 / 2 + nl] = gate_mul(a.act, g, u);
                 }
             }
         }
@@ -495,7 +495,7 @@ __global__ __launch_bounds__(256) void gemv_kernel(GemvArgs a) {
     const int K = a.K, KC = K >> 3;
     const T* __restrict__ X = reinterpret_cast<const T*>(a.X);
     const T* __restrict__ W = reinterpret_cast<const T*>(a.W);
-    const bool silu = a.act == kActSiluMul;
+    const bool silu = act_gated(a.act);
 
     // rows this wave owns
     const int slot0 = (blockIdx.x * 4 + wave) * R;            // first "row slot"
@@ -599,7 +599,7 @@ __global__ __launch_bounds__(256) void gemv_kernel(GemvArgs a) {
             for (int mb = 0; mb < MB; ++mb) {
                 float g = acc[r][mb], u = acc[r + 1][mb];
                 if (bias) { g += to_f32(bias[rows[r]]); u += to_f32(bias[rows[r + 1]]); }
-                C[(size_t)mb * a.ldc + j] = from_f32<T>(act_silu(g) * u);
+                C[(size_t)mb * a.ldc + j] = from_f32<T>(gate_mul(a.act, g, u));
             }
         }
         return;
@@ -659,7 +659,7 @@ template <typename T, int BM, int BN, int WM, int WN, int NSTAGE, int BK = 64, i
 static void launch_gemm_pipe(const GemmArgs& a, hipStream_t st) {
     constexpr int smem = KS * NSTAGE * (BM + BN) * BK * 2;
     static_assert(smem <= 160 * 1024, "LDS ring does not fit");
-    if (a.act == kActSiluMul) LMX_REQUIRE((BN / WN / 32) % 2 == 0, "gemm: this tile cannot pair gate/up rows (SiLU·mul needs an even number of 32-wide n tiles per wave)");
+    if (act_gated(a.act)) LMX_REQUIRE((BN / WN / 32) % 2 == 0, "gemm: this tile cannot pair gate/up rows (SiLU·mul needs an even number of 32-wide n tiles per wave)");
     auto kern = gemm_pipe_kernel<T, BM, BN, WM, WN, NSTAGE, BK, KS>;
     static bool attr_set = false;
     if (!attr_set) {
@@ -698,7 +698,7 @@ static void launch_gemm16(const GemmArgs& a, int variant, hipStream_t st) {
                                                                // tiles (o_proj 58 vs 64 us, down_proj 146 vs 152 us at T=1087; TP-rank shapes
                                                                // 1087x3072x4096 44 vs 52 us, 1087x2816x4096 46 vs 51 us: profiles/EXPERIMENTS.md)
         else if (t128x256 >= 128) variant = 7;                 // 128x256, 3-slot ring   (o_proj, down_proj)
-        else if (t64 <= 320 && a.act != kActSiluMul) {                  // (<= : CLIP fc1 577 x 4096 x 1024 has exactly 320 -> 64x64 2-slot kernel, 14.6 vs 16.5 us for 64x128)
+        else if (t64 <= 320 && !act_gated(a.act)) {                  // (<= : CLIP fc1 577 x 4096 x 1024 has exactly 320 -> 64x64 2-slot kernel, 14.6 vs 16.5 us for 64x128)
             // CLIP-sized problems are latency-bound: with few 64x64 tiles (<= 2 per CU) keep three K-slabs in flight per
             // workgroup (4-slot ring, 64 KB LDS); with more tiles the 2-slot kernel's higher occupancy (32 KB) wins.
             const long t64x64 = (long)cdiv(a.M, 64) * cdiv(a.N, 64);
@@ -711,13 +711,13 @@ static void launch_gemm16(const GemmArgs& a, int variant, hipStream_t st) {
     switch (variant) {
         case 2: launch_gemm_cfg<T, 128, 128, 2, 2, false>(a, st); break;
         case 4: launch_gemm_cfg<T, 64, 128, 2, 2, true>(a, st); break;
-        case 5: LMX_REQUIRE(a.act != kActSiluMul, "gemm: the 64x64 tile has no SiLU·mul epilogue"); launch_gemm_cfg<T, 64, 64, 2, 2, true>(a, st); break;
+        case 5: LMX_REQUIRE(!act_gated(a.act), "gemm: the 64x64 tile has no SiLU·mul epilogue"); launch_gemm_cfg<T, 64, 64, 2, 2, true>(a, st); break;
         case 7: launch_gemm_pipe<T, 128, 256, 2, 4, 3>(a, st); break;          // 128x256x64, 3-slot ring (two slabs in flight)
         case 9: launch_gemm_pipe<T, 256, 256, 2, 4, 2>(a, st); break;          // 256x256x64, 2-slot ring, 128 FLOP per L2 byte
-        case 15: LMX_REQUIRE(a.act != kActSiluMul, "gemm: the 64x64 tile has no SiLU·mul epilogue"); launch_gemm_pipe<T, 64, 64, 2, 2, 4>(a, st); break;   // small tiles, 4 waves, 4-slot ring: latency-bound shapes
+        case 15: LMX_REQUIRE(!act_gated(a.act), "gemm: the 64x64 tile has no SiLU·mul epilogue"); launch_gemm_pipe<T, 64, 64, 2, 2, 4>(a, st); break;   // small tiles, 4 waves, 4-slot ring: latency-bound shapes
         // in-workgroup split-K forms of the same tile (round 5): 16 = 2 groups x 4-slot rings (128 KB), 17 = 4 groups x 2-slot rings (128 KB, 16 waves)
-        case 16: LMX_REQUIRE(a.act != kActSiluMul, "gemm: the 64x64 tile has no SiLU·mul epilogue"); launch_gemm_pipe<T, 64, 64, 2, 2, 4, 64, 2>(a, st); break;
-        case 17: LMX_REQUIRE(a.act != kActSiluMul, "gemm: the 64x64 tile has no SiLU·mul epilogue"); launch_gemm_pipe<T, 64, 64, 2, 2, 2, 64, 4>(a, st); break;
+        case 16: LMX_REQUIRE(!act_gated(a.act), "gemm: the 64x64 tile has no SiLU·mul epilogue"); launch_gemm_pipe<T, 64, 64, 2, 2, 4, 64, 2>(a, st); break;
+        case 17: LMX_REQUIRE(!act_gated(a.act), "gemm: the 64x64 tile has no SiLU·mul epilogue"); launch_gemm_pipe<T, 64, 64, 2, 2, 2, 64, 4>(a, st); break;
         // N = hidden-size outputs at T ~ 1k (o_proj, down_proj) without split-K scratch and the tensor-parallel rank shapes: 128x128 gives 288 workgroups small
         // enough (64 KB LDS) for two to share a CU, so every CU has work for the whole kernel.
         case 18: launch_gemm_pipe<T, 128, 128, 2, 2, 2>(a, st); break;
@@ -749,8 +749,8 @@ void launch_gemm(int dtype, const GemmArgs& a, int variant, hipStream_t st) {
         return;
     }
     LMX_REQUIRE(a.N % 8 == 0, "gemm: N must be a multiple of 8");
-    LMX_REQUIRE(!a.c_f32 || (!a.skw && !a.pk_kc && !a.qf_kc && !a.R && a.act != kActSiluMul), "gemm: fp32 output is for plain un-split linears");
-    if (a.act == kActSiluMul) LMX_REQUIRE(a.N % 64 == 0, "gemm: SiLU·mul needs N (fused gate|up rows) % 64 == 0");
+    LMX_REQUIRE(!a.c_f32 || (!a.skw && !a.pk_kc && !a.qf_kc && !a.R && !act_gated(a.act)), "gemm: fp32 output is for plain un-split linears");
+    if (act_gated(a.act)) LMX_REQUIRE(a.N % 64 == 0, "gemm: SiLU·mul needs N (fused gate|up rows) % 64 == 0");
     if (dtype == kF32) {
         LMX_REQUIRE(a.K % 16 == 0, "gemm f32: K must be a multiple of 16");
         const int mtiles = cdiv(a.M, 64), ntiles = cdiv(a.N, 64);
@@ -821,8 +821,8 @@ bool gemv_residual_applies(int dtype, const GemvArgs& a) {
 }
 void launch_gemv_residual(int dtype, GemvArgs a, const ResidualNormArgs& rn, hipStream_t st) {
     LMX_REQUIRE(gemv_residual_applies(dtype, a), "gemv_residual: 16-bit weights, 16-byte rows, K up to 8192");
-    LMX_REQUIRE(rn.H == a.K && rn.pre_w && rn.x_out && rn.x_out != rn.x_in && (!rn.y || rn.post_w) && (rn.y || rn.inject || rn.x_in), "gemv_residual: bad residual arguments (x_out must be another row than x_in)");
-    LMX_REQUIRE(!a.R && (a.act != kActSiluMul || a.N % 64 == 0), "gemv_residual: no second residual; SiLU*mul needs N % 64 == 0");
+    LMX_REQUIRE(rn.H == a.K && rn.pre_w && rn.x_out && rn.x_out != rn.x_in && rn.top == 0 && !rn.cast && (rn.y || rn.inject || rn.x_in), "gemv_residual: bad residual arguments (x_out must be another row than x_in)");
+    LMX_REQUIRE(!a.R && (!act_gated(a.act) || a.N % 64 == 0), "gemv_residual: no second residual; SiLU*mul needs N % 64 == 0");
     a.X = rn.y; a.norm_w = rn.pre_w;
     if (dtype == kBF16) launch_gemv2_res<bf16_t>(a, rn, st); else launch_gemv2_res<f16_t>(a, rn, st);
 }
@@ -835,7 +835,7 @@ static bool launch_gemv2(const GemvArgs& a, hipStream_t st) {
     if constexpr (sizeof(T) != 2) return false;
     else {
         if (!gemv2_applies(TypeInfo<T>::id, a)) return false;
-        if (a.act == kActSiluMul) launch_gemv2_r<T, 2, 4>(a, st);
+        if (act_gated(a.act)) launch_gemv2_r<T, 2, 4>(a, st);
         else if (a.K >= 8192) launch_gemv2_r<T, 1, 8>(a, st);
         // small linears (<= 32 M weights): o_proj keeps one row per wave (1024 short-lived workgroups); with the RMSNorm fused — the split-q step's q projection — every
         // workgroup also normalises the whole input row, so half as many workgroups with two rows per wave win: 8.1 -> 7.5 us (profiles/r05_small_gemv_rp.txt)
@@ -851,7 +851,7 @@ static void launch_gemv_mb(const GemvArgs& a, hipStream_t st) {
     // R weight rows per wave: more rows = more independent 16-byte loads in flight per lane, fewer = more workgroups.
     // cold-cache sweep (tools/mb_gemv_cold.py, 7B shapes): o_proj 8.8 us at R=1 vs 9.9 at R=2; gate|up 31.3 at R=2 vs 32.5 at R=4;
     // qkv / down / lm_head are flat between R=2 and R=4; R=8 loses everywhere (too few workgroups).
-    const int R = a.act == kActSiluMul ? 2 : ((size_t)a.N * a.K <= ((size_t)1 << 24) ? 1 : (a.N >= 8192 ? 4 : 2));      // SiLU·mul pairs a gate row with its up row inside one wave
+    const int R = act_gated(a.act) ? 2 : ((size_t)a.N * a.K <= ((size_t)1 << 24) ? 1 : (a.N >= 8192 ? 4 : 2));      // SiLU·mul pairs a gate row with its up row inside one wave
     if (R == 4) launch_gemv_r<T, MB, 4>(a, st);
     else if (R == 2) launch_gemv_r<T, MB, 2>(a, st);
     else launch_gemv_r<T, MB, 1>(a, st);
@@ -871,7 +871,7 @@ static void launch_gemv_t(const GemvArgs& a, int MB, hipStream_t st) {
 void launch_gemv(int dtype, const GemvArgs& a, int MB, hipStream_t st) {
     LMX_REQUIRE(a.K % 8 == 0, "gemv: K must be a multiple of 8");
     LMX_REQUIRE((size_t)MB * a.K * dtype_size(dtype) + 16 <= 160 * 1024, "gemv: x does not fit LDS");
-    if (a.act == kActSiluMul) LMX_REQUIRE(a.N % 64 == 0, "gemv: SiLU·mul needs N % 64 == 0");
+    if (act_gated(a.act)) LMX_REQUIRE(a.N % 64 == 0, "gemv: SiLU·mul needs N % 64 == 0");
     if (dtype == kBF16) launch_gemv_t<bf16_t>(a, MB, st);
     else if (dtype == kF16) launch_gemv_t<f16_t>(a, MB, st);
     else if (dtype == kF32) launch_gemv_t<float>(a, MB, st);

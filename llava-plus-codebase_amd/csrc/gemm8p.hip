@@ -570,7 +570,7 @@ static void launch_gemm8p_t(GemmArgs a, hipStream_t st) {
     LMX_REQUIRE(a.K % 64 == 0, "gemm8p: K must be a multiple of 64");
     LMX_REQUIRE((size_t)a.M * a.ldx * sizeof(T) < ((size_t)1 << 32) && (size_t)a.N * a.ldw * sizeof(T) < ((size_t)1 << 32),
                 "gemm8p: operands must be addressable with 32-bit byte offsets");
-    if (a.act == kActSiluMul) LMX_REQUIRE(a.N % 64 == 0, "gemm8p: SiLU·mul needs N % 64 == 0");
+    if (act_gated(a.act)) LMX_REQUIRE(a.N % 64 == 0, "gemm8p: SiLU·mul needs N % 64 == 0");
     const int tiles = cdiv(a.M, 256) * cdiv(a.N, 256);
     int S = a.split_k > 0 ? a.split_k : gemm8p_pick_split(a.M, a.N, a.K);
     if (S > 3) S = 3;                                   // instantiated: 1, 2, 3 slices
@@ -611,14 +611,14 @@ static void launch_gemm8p_t(GemmArgs a, hipStream_t st) {
                              (a.qf_nkv * a.qf_D) % 256 == 0 && a.N == (a.qf_nh + 2 * a.qf_nkv) * a.qf_D && a.qf_pos0 % 8 == 0 && a.qf_smax % 8 == 0 && !a.bias && !a.R &&
                              a.act == kActNone && a.ldc % 8 == 0, "gemm8p: the fused q|k|v epilogue needs an un-split launch over head-aligned tiles (gemm_fuses_qkv)");
     // the CLIP K / V^T pack lives in gemm_epilogue only: the K-sliced launches' reduction kernels would write the k | v columns to C and leave the pack untouched
-    if (a.pk_kc) LMX_REQUIRE(S == 1 && a.act != kActSiluMul && a.pk_D % 4 == 0, "gemm8p: the K / V^T pack epilogue needs an un-split launch of a plain linear");
+    if (a.pk_kc) LMX_REQUIRE(S == 1 && !act_gated(a.act) && a.pk_D % 4 == 0, "gemm8p: the K / V^T pack epilogue needs an un-split launch of a plain linear");
     if (S == 3) launch(gemm8p_kernel<T, 3>);
     else if (S == 2) launch(gemm8p_kernel<T, 2>);
     else launch(gemm8p_kernel<T, 1>);
     if (two) {
         const dim3 rg(tiles * 8);
         // row-order output through LDS; SiLU.mul pairs columns 32 apart and unaligned rows keep the accumulator-order epilogue
-        const bool rows = a.act != kActSiluMul && a.N % 4 == 0 && a.ldc % 4 == 0 && (!a.R || a.ldr % 4 == 0);
+        const bool rows = !act_gated(a.act) && a.N % 4 == 0 && a.ldc % 4 == 0 && (!a.R || a.ldr % 4 == 0);
         auto red = [&](auto kern) {
             if (timed) hipExtLaunchKernelGGL(kern, rg, dim3(256), 0, st, nullptr, kt->e1, 0, a); else hipLaunchKernelGGL(kern, rg, dim3(256), 0, st, a);
             LMX_CHECK_HIP(hipGetLastError());

@@ -81,7 +81,7 @@ __device__ __forceinline__ void gemm_epilogue(const GemmArgs& a, f32x16 (&acc)[N
     const T* R = reinterpret_cast<const T*>(a.R);
     const int act = a.act;
 
-    if (act == kActSiluMul) {
+    if (act_gated(act)) {
         // fused rows are interleaved [32 gate | 32 up] per 64: tile i even = gate, i+1 = up, same lane/register
         if constexpr (NTL % 2 == 0) {
 #pragma unroll
@@ -104,7 +104,7 @@ __device__ __forceinline__ void gemm_epilogue(const GemmArgs& a, f32x16 (&acc)[N
                             g += to_f32(bias[nfused + 8 * q + 4 * hi + e]);
                             u += to_f32(bias[nfused + 32 + 8 * q + 4 * hi + e]);
                         }
-                        v[e] = act_silu(g) * u;
+                        v[e] = gate_mul(act, g, u);
                     }
                     store4<T>(C + (size_t)m * a.ldc + no, v);
                 }

@@ -34,7 +34,7 @@ __device__ __forceinline__ void gemv2_body(const GemvArgs& a, int bid, char* sme
     const int K = a.K, KC = K >> 3;
     const int NR = (KC + 63) >> 6;                            // load rounds per row
     const T* __restrict__ X = reinterpret_cast<const T*>(a.X);
-    const bool silu = a.act == kActSiluMul;
+    const bool silu = act_gated(a.act);
 
     const int slot0 = (bid * 4 + wave) * R;            // first "row slot" of this wave
     int rows[R];
@@ -60,6 +60,7 @@ __device__ __forceinline__ void gemv2_body(const GemvArgs& a, int bid, char* sme
     //      the first P weight rounds are still on the wire.  (As plain loads behind the weight issue its wait was a vmcnt(0): staging started only after
     //      the first P rounds had landed too.)
     const bool has_x = !RES || a.X != nullptr;                // RES: the first linear of a step has no sublayer output in front of it
+    const bool has_post = RES && has_x && rn->post_w != nullptr;
     const ws_v4i rsX = ws_make_rsrc(has_x ? a.X : a.W, 0x7fffffffu);
     ws_u32x4 xraw[GEMV2_NX];
     if (has_x) {
@@ -71,13 +72,13 @@ __device__ __forceinline__ void gemv2_body(const GemvArgs& a, int bid, char* sme
     }
     ws_u32x4 praw[RES ? GEMV2_NX : 1], iraw[RES ? GEMV2_NX : 1], r0raw[RES ? GEMV2_NX : 1], r1raw[RES ? GEMV2_NX : 1];
     if constexpr (RES) {
-        const ws_v4i rsP = ws_make_rsrc(has_x ? rn->post_w : a.W, 0x7fffffffu), rsI = ws_make_rsrc(rn->inject ? rn->inject : a.W, 0x7fffffffu),
+        const ws_v4i rsP = ws_make_rsrc(has_post ? rn->post_w : a.W, 0x7fffffffu), rsI = ws_make_rsrc(rn->inject ? rn->inject : a.W, 0x7fffffffu),
                      rsR0 = ws_make_rsrc(rn->x_in ? static_cast<const void*>(rn->x_in) : a.W, 0x7fffffffu);
 #pragma unroll
         for (int i = 0; i < GEMV2_NX; ++i) {
             const int c = tid + 256 * i;
             if (c >= KC) continue;
-            if (has_x) ws_load_plain(praw[i], (uint32_t)c * 16u, rsP, 0u);
+            if (has_post) ws_load_plain(praw[i], (uint32_t)c * 16u, rsP, 0u);
             if (rn->inject) ws_load_plain(iraw[i], (uint32_t)c * 16u, rsI, 0u);
             if (rn->x_in) { ws_load_plain(r0raw[i], (uint32_t)c * 32u, rsR0, 0u); ws_load_plain(r1raw[i], (uint32_t)c * 32u + 16u, rsR0, 0u); }
         }
@@ -121,7 +122,7 @@ __device__ __forceinline__ void gemv2_body(const GemvArgs& a, int bid, char* sme
                     for (int e = 0; e < 8; ++e) ss += v[e] * v[e];
                 }
             }
-            inv1 = rn->mult / sqrtf(block_sum<4>(ss, red) * rH + rn->eps);
+            inv1 = has_post ? rn->mult / sqrtf(block_sum<4>(ss, red) * rH + rn->eps) : rn->mult;
         }
         float s2 = 0.f;
 #pragma unroll
@@ -138,7 +139,11 @@ __device__ __forceinline__ void gemv2_body(const GemvArgs& a, int bid, char* sme
                 if (has_x) {
                     float v[8], g[8];
                     ws_unpack8<T>(xraw[i], v);
-                    ws_wait1<P * R>(praw[i]); ws_unpack8<T>(praw[i], g);
+                    if (has_post) { ws_wait1<P * R>(praw[i]); ws_unpack8<T>(praw[i], g); }
+                    else {
+#pragma unroll
+                        for (int e = 0; e < 8; ++e) g[e] = 1.f;
+                    }
 #pragma unroll
                     for (int e = 0; e < 8; ++e) xv[i][e] += v[e] * inv1 * g[e];
                 }
@@ -242,7 +247,7 @@ __device__ __forceinline__ void gemv2_body(const GemvArgs& a, int bid, char* sme
                 if (j >= a.N / 2) continue;
                 float g = acc[r], u = acc[r + 1];
                 if (bias) { g += to_f32(bias[rows[r]]); u += to_f32(bias[rows[r + 1]]); }
-                C[j] = from_f32<T>(act_silu(g) * u);
+                C[j] = from_f32<T>(gate_mul(a.act, g, u));
             }
         }
         return;
@@ -281,7 +286,7 @@ __device__ __forceinline__ void residual_row_store(const ResidualNormArgs& rn, f
 #pragma unroll
             for (int e = 0; e < 8; ++e) ss += v[e] * v[e];
         }
-        inv1 = rn.mult / sqrtf(block_sum<4>(ss, red) * (1.f / (float)rn.H_real) + rn.eps);
+        inv1 = post ? rn.mult / sqrtf(block_sum<4>(ss, red) * (1.f / (float)rn.H_real) + rn.eps) : rn.mult;
     }
     for (int c = tid; c < HC; c += 256) {
         float x[8], v[8], g[8];
@@ -291,9 +296,10 @@ __device__ __forceinline__ void residual_row_store(const ResidualNormArgs& rn, f
             for (int e = 0; e < 8; ++e) x[e] = 0.f;
         }
         if (y) {
-            load8<T>(y + c * 8, v); load8<T>(post + c * 8, g);
+            load8<T>(y + c * 8, v);
+            if (post) load8<T>(post + c * 8, g);
 #pragma unroll
-            for (int e = 0; e < 8; ++e) x[e] += v[e] * inv1 * g[e];
+            for (int e = 0; e < 8; ++e) x[e] += v[e] * inv1 * (post ? g[e] : 1.f);
         }
         if (inj) {
             load8<T>(inj + c * 8, g);

@@ -132,7 +132,7 @@ void launch_attn_probs(int dtype, int D, const AttnProbsArgs& a, hipStream_t st)
 // Partials (o[D], m, l) per (head, split) go to `ws`; the last workgroup to arrive for a head merges them in the same
 // launch (agent-scope counter protocol), so there is no separate combine launch.
 // decode batch (continuous batching): per-sequence pointers of ONE layer; workgroup (head, split, z) serves sequence z
-struct DecodeFusedSeq { void* K; void* VT; const int* pos_ptr; float* ws; int* counters; };
+struct DecodeFusedSeq { void* K; void* VT; const int* pos_ptr; float* ws; int* counters; const int* done = nullptr; };      // done: the sequence's stop flag (recurrent state stands still once it is set)
 struct DecodeFusedArgs {
     const void* QKV;       // [qkv_n] row of this token: q heads | k heads | v heads (pre-RoPE)
     void* K;               // caches of this layer (the new key/value are appended at *pos_ptr)
@@ -155,15 +155,30 @@ size_t decode_fused_ws_floats(int n_heads, int n_split, int D);
 size_t decode_attn_ws_floats(int n_rows, int n_heads, int n_split, int D);
 
 // ---- layer-stack decoders (stack_ops.hip) ------------------------------------------------------------------------------------------------------------------
-// x_out = x_in + mult * rms_norm(y) * post_w + inject;  xn = rms_norm(x_out) * pre_w.  Any of x_in (= 0), y, inject, x_out, pre_w may be null.  The residual stream is
-// fp32 whatever the model dtype; rows have pitch H (a multiple of 8, zero padded), the norms' means run over H_real.  x_out may be x_in.
+// x_out = x_in + mult * rms_norm(y) * post_w + inject;  xn = rms_norm(x_out) * pre_w.  Any of x_in (= 0), y, inject, x_out, pre_w may be null; without post_w the
+// sublayer output is added as it is.  The residual stream is fp32 whatever the model dtype; rows have pitch H (a multiple of 8, zero padded), the norms' means run over
+// H_real.  x_out may be x_in.  moe_y adds a mixture's expert outputs to y: y += sum_k moe_w[row][k] moe_y[row * top + k].  cast: xn = x_out in the model dtype, no norm.
 struct ResidualNormArgs {
     const float* x_in; const void* y; const void* post_w; const void* inject; const void* pre_w;
     float* x_out; void* xn;
     int H, H_real;
     float mult, eps;
+    const void* moe_y = nullptr; const float* moe_w = nullptr; int top = 0;
+    int xn_ld = 0, cast = 0;             // row pitch of xn (0: H)
 };
 void launch_residual_norm(int dtype, const ResidualNormArgs& a, int rows, hipStream_t st);
+// input rows of a model with a bigram embedding: from a portion's ids, from one sequence's state words or from a decode batch's table
+struct SeqStateRef;
+struct EmbedRowsArgs {
+    const int* ids = nullptr;            // [rows]; row 0's previous token: *prev_id, else *prev_tok, else none
+    const int* prev_id = nullptr; const int64_t* prev_tok = nullptr;
+    const int64_t* tok = nullptr;        // one row: *tok after *prev_tok
+    const SeqStateRef* tab = nullptr;    // row i: tab[i].tok after tab[i].prev
+    const void* embed = nullptr; const void* bigram = nullptr;
+    float* x = nullptr; void* x0 = nullptr; int x0_ld = 0;       // fp32 rows [rows][H]; optional copy in the model dtype
+    int H = 0, vocab = 0, buckets = 0; int64_t mul_prev = 0, mul_cur = 0;
+};
+void launch_embed_rows(int dtype, const EmbedRowsArgs& a, int rows, hipStream_t st);
 // one row: residual_norm and the linear that reads xn in ONE launch (a.X / a.norm_w come from rn; xn is never stored).  x_out must not be x_in
 bool gemv_residual_applies(int dtype, const GemvArgs& a);
 void launch_gemv_residual(int dtype, GemvArgs a, const ResidualNormArgs& rn, hipStream_t st);
@@ -176,6 +191,7 @@ struct QkvNormRopeArgs {
     const float* cos_sin;
     int T, pos0, qkv_stride, n_heads, n_kv_heads, s_max, qk_dim, rot_dims;
     float eps;
+    int zero_to = 0;                      // cache rows [pos0 + T, pos0 + zero_to) become zero (caches whose memory held something else before)
 };
 void launch_qkv_norm_rope_kv(int dtype, int D, const QkvNormRopeArgs& a, hipStream_t st);
 // attention of prompt rows on the vector ALUs (any dtype; FlashArgs' windowed causal form)
@@ -193,6 +209,72 @@ struct WinDecodeArgs {
     float scale = 1.f, eps = 0.f;
 };
 void launch_decode_win(int dtype, int D, const WinDecodeArgs& a, hipStream_t st);
+
+// ---- gated delta rule (delta.hip): per head a state S [key channel][value channel] in fp32, S <- g S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q -----------------
+// Projection rows of a layer: q [G][DK] | k [G][DK] | v [H][DV] | beta [H] | ...; DK in {64, 128, 256} and DV (a multiple of 64) are padded head widths, the padding is
+// zero.  q, k, v pass a causal convolution of `taps` inputs per channel and silu; q and k are unit vectors; the decay is one per head and key channel.
+// State of a sequence and layer run: S transposed, [H][DV][DK] floats, and a ring of the last `taps` projection rows (row of position p at p % taps), [taps][channels].
+struct DeltaShape {
+    int H = 0, G = 0, DK = 0, DV = 0, dk = 0, dv = 0, taps = 1;      // heads, key heads, padded and true widths
+    __host__ __device__ int channels() const { return 2 * G * DK + H * DV; }
+    size_t state_floats() const { return (size_t)H * DV * DK; }
+};
+struct DeltaWeights { const void* conv; const void* A_log; const void* dt_bias; const void* norm; };      // conv [taps][channels], A_log [H], dt_bias [H][DK], norm [DV]
+constexpr int DELTA_MAX_SEG = 16;
+struct DeltaSeg { int row0, n, pos0; float* state; void* ring; };        // rows [row0, row0 + n) of the piece continue a sequence at position pos0 (0: from a zero state)
+struct DeltaPrefillArgs {
+    DeltaShape s; DeltaWeights w;
+    const void* proj; int ld;            // projection rows
+    const void* ag; int ag_ld;           // decay pre-activations [H][DK] | output gates [H][DV]
+    float* qk; float* g; void* v; float* sc; float* o;      // scratch rows: [G][2][DK] unit q, k | [H][DK] decays | [H][DV] | [H] {beta, q . k} pairs | [H][DV]
+    void* out; int out_ld;               // [H][DV] rows
+    float eps;
+    int n_seg; DeltaSeg seg[DELTA_MAX_SEG];
+};
+size_t delta_scratch_bytes(const DeltaShape& s, int rows, int es);
+void delta_carve(DeltaPrefillArgs& a, void* scratch, int rows, int es);
+void launch_delta_prep(int dtype, const DeltaPrefillArgs& a, hipStream_t st);      // convolutions, unit norms, decays, step sizes
+void launch_delta_scan(int dtype, const DeltaPrefillArgs& a, hipStream_t st);      // the recurrence; leaves state and ring behind
+void launch_delta_gate(int dtype, const DeltaPrefillArgs& a, hipStream_t st);      // root-mean-square norm and output gate
+struct DeltaDecodeArgs {                 // one new token per sequence, everything in one launch
+    DeltaShape s; DeltaWeights w;
+    const void* proj; int ld; int a_off, ra, rg;            // columns a_off: [ra] decay latent | [rg] gate latent
+    const void* wag; int wag_ld;         // [H * DK] decay rows (first ra columns) | [H * DV] gate rows (the rg columns behind)
+    void* out; int out_ld;
+    const DecodeFusedSeq* tab = nullptr; DecodeFusedSeq one{};      // K = state, VT = ring
+    int n_seq = 1;
+    float eps;
+};
+void launch_delta_decode(int dtype, const DeltaDecodeArgs& a, hipStream_t st);
+
+// ---- latent attention (latent.hip): keys and values are linear in a normalised latent row, the only thing that is cached: [s_max][R] ---------------------------------
+struct LatentNormArgs {                  // rows: c_q <- rms_norm(c_q) in place, cache[pos] <- rms_norm(c)
+    void* proj; int ld, Q, q_n, R, r_n;  // c_q at column 0 (Q padded, q_n true), c at column Q
+    const void* q_w; const void* r_w;
+    void* cache; int pos0;               // row i goes to position pos0 + i; with tab: one row per sequence at *pos_ptr (cache = K)
+    const DecodeFusedSeq* tab = nullptr; const int* pos_ptr = nullptr;
+    int s_max; float eps;
+};
+void launch_latent_norm(int dtype, const LatentNormArgs& a, int rows, hipStream_t st);
+struct LatentDecodeArgs {                // queries already in the latent space, [n_seq][H][R]; out the attention-weighted latents, same layout
+    const void* q; void* out;
+    const DecodeFusedSeq* tab = nullptr; DecodeFusedSeq one{};
+    int n_seq = 1, H = 0, R = 0, s_max = 0, n_split = 1, window = 0;
+    float scale = 1.f;
+};
+void launch_latent_decode(int dtype, const LatentDecodeArgs& a, hipStream_t st);
+
+// ---- grouped linears and mixtures of experts (moe.hip) -----------------------------------------------------------------------------------------------------------
+struct GroupGemvArgs {                   // slot = blockIdx.y.  ids: group = ids[slot], x row slot / per_row, c row slot.  no ids: group = slot % groups, x and c row slot / groups
+    const void* X; const void* W; void* C;
+    int N, K, ldx, ldw, ldc; size_t w_group;      // w_group: elements between groups' weights
+    int x_group = 0, c_group = 0;        // no ids: element offsets per group inside the x / c rows
+    int act = 0;
+    const int* ids = nullptr; int per_row = 1, groups = 1;
+};
+void launch_group_gemv(int dtype, const GroupGemvArgs& a, int slots, hipStream_t st);
+struct MoeRouterArgs { const void* x; const void* w; const void* bias; int ldx, K, E, top; int* ids; float* wt; };      // ids / wt [rows][top]: the largest logits and their softmax
+void launch_moe_router(int dtype, const MoeRouterArgs& a, int rows, hipStream_t st);
 
 // ---- decode-step attention of a single request (decode_attn.hip; 16-bit models) ---------------------------------------------------------------------
 // RoPE(q, k_new) + KV append + attention over 128-key chunks + in-launch merge, position BY VALUE (the engine mirrors *d_len on the host), only the live
@@ -281,7 +363,7 @@ struct SampleParams { float temperature = 0.f; float top_p = 1.f; int top_k = 0;
 // batch still running — produce nothing past the stop and the host needs no per-token round trip to know where it was.
 constexpr int STOP_MAX_EOS = 4, STOP_MAX_KW = 4, STOP_MAX_KW_LEN = 8;
 struct StopSpec { int done; int n_eos; int n_kw; int pad; int64_t eos[STOP_MAX_EOS]; int kw_len[STOP_MAX_KW]; int64_t kw[STOP_MAX_KW][STOP_MAX_KW_LEN]; };
-struct SeqStateRef { int* len; int* n_out; int64_t* tok; int64_t* log; int log_cap; int pad; SampleParams sample; StopSpec* stop; };
+struct SeqStateRef { int* len; int* n_out; int64_t* tok; int64_t* log; int log_cap; int pad; SampleParams sample; StopSpec* stop; int64_t* prev = nullptr; };      // prev: the token the step just fed
 // the two id rules on a sequence whose n_after generated ids (the last one = t) sit in log[0 .. n_after): t is an EOS id | the last len(kw) ids equal kw
 __device__ __forceinline__ bool stop_rule_fires(const StopSpec* sp, int64_t t, const int64_t* log, int n_after, int log_cap) {
     bool hit = false;

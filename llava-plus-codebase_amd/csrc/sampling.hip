@@ -379,6 +379,7 @@ __global__ __launch_bounds__(CPT > 0 ? FAST_NT : 1024) void pick_advance_batch_k
         t = idx == 0x7fffffff ? 0 : idx;
     }
     if (threadIdx.x == 0) {
+        if (r.prev) *r.prev = *r.tok;                       // the token this step fed
         *r.tok = t;
         if (ids_out) ids_out[blockIdx.x] = t;
         *r.len += 1;

@@ -70,7 +70,7 @@ __global__ __launch_bounds__(NW * 64) void skinny_gemm_kernel(GemmArgs a) {
 
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
     const int i = lane & 15, q = lane >> 4;
-    const bool silu = a.act == kActSiluMul;
+    const bool silu = act_gated(a.act);
     const int K = a.K;
 
     int rowbase[RT];
@@ -275,7 +275,7 @@ __global__ __launch_bounds__(NW * 64) void skinny_gemm_kernel(GemmArgs a) {
             if (m >= a.M || j >= a.N / 2) continue;
             float g = tile_sum(gi * CT + ct, token, nrow), u = tile_sum((gi + HALF) * CT + ct, token, nrow);
             if (bias) { g += to_f32(bias[rowbase[gi] + nrow]); u += to_f32(bias[rowbase[gi + HALF] + nrow]); }
-            C[(size_t)m * a.ldc + j] = from_f32<T>(act_silu(g) * u);
+            C[(size_t)m * a.ldc + j] = from_f32<T>(gate_mul(a.act, g, u));
         }
         return;
     }
@@ -308,7 +308,7 @@ size_t skinny_scratch_bytes(int N) { return (size_t)cdiv(N, 64) * 8 * (4 * 2 * 2
 template <typename T, bool SWZ>
 static void launch_skinny_s(const GemmArgs& a, hipStream_t st) {
     constexpr int NW = 8;
-    const bool silu = a.act == kActSiluMul;
+    const bool silu = act_gated(a.act);
     const int ct = a.M > 16 ? 2 : 1;
     // the fragment-order copy with whole 128-k super-steps takes the hand-counted load stream; same tile forms, same bits
     const bool stream = SWZ && a.K % SK_SUPER == 0;
@@ -376,7 +376,7 @@ void launch_skinny_gemm(int dtype, const GemmArgs& a, hipStream_t st) {
     LMX_REQUIRE(a.M >= 1 && a.M <= 32, "skinny gemm: 1..32 token rows");
     LMX_REQUIRE(a.N > 0 && a.K > 0 && a.K % 32 == 0, "skinny gemm: K must be a multiple of 32");
     LMX_REQUIRE(a.ldx % 8 == 0 && a.ldw % 8 == 0, "skinny gemm: leading dims must keep 16-byte row alignment");
-    if (a.act == kActSiluMul) LMX_REQUIRE(a.N % 64 == 0, "skinny gemm: SiLU·mul needs N (fused gate|up rows) % 64 == 0");
+    if (act_gated(a.act)) LMX_REQUIRE(a.N % 64 == 0, "skinny gemm: SiLU·mul needs N (fused gate|up rows) % 64 == 0");
     if (dtype == kBF16) launch_skinny_t<bf16_t>(a, st); else launch_skinny_t<f16_t>(a, st);
 }
 

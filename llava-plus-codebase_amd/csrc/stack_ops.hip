@@ -26,7 +26,7 @@ __global__ __launch_bounds__(256) void residual_norm_kernel(ResidualNormArgs a) 
     const float* xin = a.x_in ? a.x_in + (size_t)row * a.H : nullptr;
     const T* y = a.y ? reinterpret_cast<const T*>(a.y) + (size_t)row * a.H : nullptr;
     const T* inj = a.inject ? reinterpret_cast<const T*>(a.inject) + (size_t)row * a.H : nullptr;
-    const T* post = reinterpret_cast<const T*>(a.post_w);
+    const T* post = y || a.top > 0 ? reinterpret_cast<const T*>(a.post_w) : nullptr;
     const T* pre = reinterpret_cast<const T*>(a.pre_w);
     float x[NP][8], yv[NP][8];
     float ss = 0.f;
@@ -39,13 +39,26 @@ __global__ __launch_bounds__(256) void residual_norm_kernel(ResidualNormArgs a) 
 #pragma unroll
             for (int e = 0; e < 8; ++e) x[i][e] = 0.f;
         }
-        if (y) {
-            load8<T>(y + c * 8, yv[i]);
+        if (y) load8<T>(y + c * 8, yv[i]);
+        else {
+#pragma unroll
+            for (int e = 0; e < 8; ++e) yv[i][e] = 0.f;
+        }
+        for (int k = 0; k < a.top; ++k) {
+            const float wk = a.moe_w[(size_t)row * a.top + k];
+            float v[8]; load8<T>(reinterpret_cast<const T*>(a.moe_y) + ((size_t)row * a.top + k) * a.H + c * 8, v);
+#pragma unroll
+            for (int e = 0; e < 8; ++e) yv[i][e] = fmaf(wk, v[e], yv[i][e]);
+        }
+        if (post) {
 #pragma unroll
             for (int e = 0; e < 8; ++e) ss += yv[i][e] * yv[i][e];
+        } else {
+#pragma unroll
+            for (int e = 0; e < 8; ++e) x[i][e] += a.mult * yv[i][e];
         }
     }
-    if (y) {
+    if (post) {
         ss = block_sum<4>(ss, red);
         const float inv = a.mult / sqrtf(ss * rH + a.eps);
 #pragma unroll
@@ -71,10 +84,15 @@ __global__ __launch_bounds__(256) void residual_norm_kernel(ResidualNormArgs a) 
 #pragma unroll
         for (int e = 0; e < 8; ++e) s2 += x[i][e] * x[i][e];
     }
+    T* xn = reinterpret_cast<T*>(a.xn) + (size_t)row * (a.xn_ld ? a.xn_ld : a.H);
+    if (a.cast) {
+#pragma unroll
+        for (int i = 0; i < NP; ++i) { const int c = tid + i * 256; if (c < HC) store8<T>(xn + c * 8, x[i]); }
+        return;
+    }
     if (!pre) return;
     s2 = block_sum<4>(s2, red);
     const float inv2 = 1.f / sqrtf(s2 * rH + a.eps);
-    T* xn = reinterpret_cast<T*>(a.xn) + (size_t)row * a.H;
 #pragma unroll
     for (int i = 0; i < NP; ++i) {
         const int c = tid + i * 256;
@@ -86,10 +104,55 @@ __global__ __launch_bounds__(256) void residual_norm_kernel(ResidualNormArgs a) 
     }
 }
 
+// ---------------------------------------------------------------------------------------------------------------
+// input rows of a model whose embedding depends on the token before: x = embed[t] + bigram[(prev mul_prev + t mul_cur) mod buckets] (row `buckets` without a previous
+// token), summed in fp32.  One workgroup per row.
+// ---------------------------------------------------------------------------------------------------------------
+template <typename T>
+__global__ __launch_bounds__(256) void embed_rows_kernel(EmbedRowsArgs a) {
+    const int row = blockIdx.x, tid = threadIdx.x;
+    int64_t t, prev = -1;
+    if (a.tab) { t = *a.tab[row].tok; prev = *a.tab[row].prev; }
+    else if (a.ids) {
+        t = a.ids[row];
+        if (row > 0) prev = a.ids[row - 1];
+        else if (a.prev_id) prev = *a.prev_id;
+        else if (a.prev_tok) prev = *a.prev_tok;
+    } else { t = *a.tok; prev = *a.prev_tok; }
+    t = t < 0 ? 0 : (t >= a.vocab ? a.vocab - 1 : t);
+    int64_t b = a.buckets;
+    if (prev >= 0) {
+        b = (prev * a.mul_prev + t * a.mul_cur) % a.buckets;
+        if (b < 0) b += a.buckets;
+    }
+    const T* e = reinterpret_cast<const T*>(a.embed) + (size_t)t * a.H;
+    const T* g = reinterpret_cast<const T*>(a.bigram) + (size_t)b * a.H;
+    for (int c = tid; c < (a.H >> 3); c += 256) {
+        float v[8], u[8];
+        load8<T>(e + c * 8, v); load8<T>(g + c * 8, u);
+#pragma unroll
+        for (int i = 0; i < 8; ++i) v[i] += u[i];
+        store8<float>(a.x + (size_t)row * a.H + c * 8, v);
+        if (a.x0) store8<T>(reinterpret_cast<T*>(a.x0) + (size_t)row * a.x0_ld + c * 8, v);
+    }
+}
+
+void launch_embed_rows(int dtype, const EmbedRowsArgs& a, int rows, hipStream_t st) {
+    LMX_REQUIRE(a.embed && a.bigram && a.x && a.buckets >= 1 && a.H % 8 == 0 && a.vocab >= 1, "embed_rows: bad arguments");
+    LMX_REQUIRE(a.tab || a.ids || (rows == 1 && a.tok && a.prev_tok), "embed_rows: no tokens");
+    LMX_REQUIRE(!a.x0 || a.x0_ld % 8 == 0, "embed_rows: bad pitch");
+    if (rows <= 0) return;
+#define L(TT) LMX_LAUNCH(embed_rows_kernel<TT>, dim3(rows), dim3(256), 0, st, a)
+    if (dtype == kBF16) L(bf16_t); else if (dtype == kF16) L(f16_t); else L(float);
+#undef L
+    LMX_CHECK_HIP(hipGetLastError());
+}
+
 void launch_residual_norm(int dtype, const ResidualNormArgs& a, int rows, hipStream_t st) {
     LMX_REQUIRE(a.H % 8 == 0 && a.H > 0 && a.H <= 8192 && a.H_real >= 1 && a.H_real <= a.H, "residual_norm: width must be a multiple of 8, at most 8192");
-    LMX_REQUIRE(!a.y || a.post_w, "residual_norm: a sublayer output needs its norm's weight");
-    LMX_REQUIRE(!a.pre_w || a.xn, "residual_norm: the normalised rows need a buffer");
+    LMX_REQUIRE(a.top >= 0 && (a.top == 0 || (a.moe_y && a.moe_w)), "residual_norm: expert outputs need their weights");
+    LMX_REQUIRE((!a.pre_w && !a.cast) || a.xn, "residual_norm: the normalised rows need a buffer");
+    LMX_REQUIRE(!(a.pre_w && a.cast) && a.xn_ld % 8 == 0, "residual_norm: norm or cast, in 16-byte rows");
     if (rows <= 0) return;
     const int np = (a.H / 8 + 255) / 256;
 #define R(TT, NPV) LMX_LAUNCH((residual_norm_kernel<TT, NPV>), dim3(rows), dim3(256), 0, st, a)
@@ -111,7 +174,8 @@ __global__ __launch_bounds__(256) void qkv_norm_rope_kv_kernel(QkvNormRopeArgs a
     extern __shared__ __attribute__((aligned(16))) char smem[];
     const int tid = threadIdx.x;
     const int tok0 = blockIdx.x * 64, slot = blockIdx.y;
-    const int ntok = (a.T - tok0) < 64 ? (a.T - tok0) : 64;
+    const int ntok = (a.T - tok0) < 64 ? (a.T - tok0) : 64;                // <= 0: a block of nothing but rows to clear
+    const int nzero = (a.zero_to - tok0) < 64 ? (a.zero_to - tok0) : 64;
     T* qkv = reinterpret_cast<T*>(a.qkv);
     constexpr int LPV = D / 8, VPP = 256 / LPV;          // lanes per vector, vectors per pass
     if (PAIRED && slot < a.n_heads + a.n_kv_heads) {
@@ -126,7 +190,7 @@ __global__ __launch_bounds__(256) void qkv_norm_rope_kv_kernel(QkvNormRopeArgs a
 #pragma unroll
         for (int it = 0; it < ITER; ++it) {
             const int t = it * (256 / LP) + tid / LP;
-            const T* xp = qkv + (size_t)(tok0 + (t < ntok ? t : 0)) * a.qkv_stride + slot * D;
+            const T* xp = qkv + (size_t)(t < ntok ? tok0 + t : a.T - 1) * a.qkv_stride + slot * D;
             load8<T>(xp + c0 * 8, x[it][0]); load8<T>(xp + c1 * 8, x[it][1]);
         }
         if (nw) { load8<T>(nw + c0 * 8, g0); load8<T>(nw + c1 * 8, g1); }
@@ -146,8 +210,13 @@ __global__ __launch_bounds__(256) void qkv_norm_rope_kv_kernel(QkvNormRopeArgs a
 #pragma unroll
                 for (int e = 0; e < 8; ++e) { u[e] *= inv * g0[e]; v[e] *= inv * g1[e]; }
             }
-            if (!live) continue;
             const int pos = a.pos0 + tok0 + t;
+            if (!live && is_k && t < nzero) {
+#pragma unroll
+                for (int e = 0; e < 8; ++e) { u[e] = 0.f; v[e] = 0.f; }
+                store8<T>(kc + (size_t)pos * D + c0 * 8, u); store8<T>(kc + (size_t)pos * D + c1 * 8, v);
+            }
+            if (!live) continue;
             if (rot) {
                 const float* cs = a.cos_sin + (size_t)pos * a.rot_dims + k * 8;
                 float c[8], s[8];
@@ -218,9 +287,9 @@ __global__ __launch_bounds__(256) void qkv_norm_rope_kv_kernel(QkvNormRopeArgs a
     __syncthreads();
     T* vt = reinterpret_cast<T*>(a.VT) + (size_t)kvh * D * a.s_max;
     const int t = tid & 63;
-    if (t < ntok) {
+    if (t < ntok || t < nzero) {
         const int pos = a.pos0 + tok0 + t;
-        for (int d = tid >> 6; d < D; d += 4) vt[(size_t)d * a.s_max + pos] = tile[t * PITCH + d];
+        for (int d = tid >> 6; d < D; d += 4) vt[(size_t)d * a.s_max + pos] = t < ntok ? tile[t * PITCH + d] : from_f32<T>(0.f);
     }
 }
 
@@ -228,10 +297,11 @@ void launch_qkv_norm_rope_kv(int dtype, int D, const QkvNormRopeArgs& a, hipStre
     LMX_REQUIRE(D == 64 || D == 128 || D == 256, "qkv_norm_rope_kv: padded head width must be 64, 128 or 256");
     LMX_REQUIRE(a.qkv_stride % 8 == 0 && a.qkv_stride >= (a.n_heads + 2 * a.n_kv_heads) * D, "qkv_norm_rope_kv: bad row pitch");
     LMX_REQUIRE(a.rot_dims % 2 == 0 && a.rot_dims <= a.qk_dim && a.qk_dim <= D && (a.rot_dims == 0 || a.cos_sin), "qkv_norm_rope_kv: bad rotation");
-    LMX_REQUIRE(a.pos0 >= 0 && a.pos0 + a.T <= a.s_max, "qkv_norm_rope_kv: rows past the cache");
+    LMX_REQUIRE(a.pos0 >= 0 && a.pos0 + a.T <= a.s_max && a.pos0 + a.zero_to <= a.s_max, "qkv_norm_rope_kv: rows past the cache");
     if (a.T <= 0) return;
-    const dim3 grid(cdiv(a.T, 64), a.n_heads + 2 * a.n_kv_heads);
+    const dim3 grid(cdiv(a.zero_to > a.T ? a.zero_to : a.T, 64), a.n_heads + 2 * a.n_kv_heads);
     const bool paired = a.rot_dims % 16 == 0;
+    LMX_REQUIRE(a.zero_to == 0 || (paired && a.n_heads == 0), "qkv_norm_rope_kv: clearing is for key / value rows of whole rotation groups");
     size_t smem = (size_t)64 * (D + 2) * dtype_size(dtype);
     if (!paired && smem < 256 * 8 * sizeof(float)) smem = 256 * 8 * sizeof(float);
 #define L(TT, DD) do {                                                                                                                   \

@@ -12,9 +12,10 @@ from ctypes import POINTER, Structure, c_char_p, c_float, c_int32, c_int64, c_si
 _HERE = os.path.dirname(os.path.abspath(__file__))
 LIB_PATH = os.path.join(_HERE, "libllava_mi355x.so")
 
-LMX_ABI_VERSION = 1
+LMX_ABI_VERSION = 2
 DTYPE_F32, DTYPE_BF16, DTYPE_F16 = 0, 1, 2
-ACT_NONE, ACT_QUICK_GELU, ACT_GELU_ERF, ACT_SILU_MUL = 0, 1, 2, 3
+ACT_NONE, ACT_QUICK_GELU, ACT_GELU_ERF, ACT_SILU_MUL, ACT_RELU_MUL = 0, 1, 2, 3, 4
+MIXER_ATTENTION, MIXER_LATENT, MIXER_DELTA = 0, 1, 2
 PROJ_LINEAR, PROJ_MLP_GELU, PROJ_IDENTITY = 0, 1, 2
 FEATURE_PATCH, FEATURE_CLS_PATCH = 0, 1
 
@@ -38,13 +39,16 @@ class LmxConfig(Structure):
 
 class LmxLayerConfig(Structure):
     _fields_ = [("n_heads", c_int32), ("n_kv_heads", c_int32), ("qk_dim", c_int32), ("v_dim", c_int32), ("attn_scale", c_float), ("window", c_int32), ("softmax_sink", c_int32),
-                ("qk_norm", c_int32), ("qkv_bias", c_int32), ("out_gate", c_int32), ("rope_dims", c_int32), ("rope_table", c_int32), ("ff", c_int32), ("reserved", c_int32 * 8)]
+                ("qk_norm", c_int32), ("qkv_bias", c_int32), ("out_gate", c_int32), ("rope_dims", c_int32), ("rope_table", c_int32), ("ff", c_int32), ("mixer", c_int32), ("parallel", c_int32), ("ff_act", c_int32),
+                ("experts", c_int32), ("top_experts", c_int32), ("q_rank", c_int32), ("kv_rank", c_int32), ("conv_taps", c_int32), ("decay_rank", c_int32), ("gate_rank", c_int32),
+                ("reserved", c_int32 * 8)]
 
 
 class LmxStackConfig(Structure):
     _fields_ = [("abi_version", c_int32), ("dtype", c_int32), ("width", c_int32), ("vocab_size", c_int32), ("n_layers", c_int32), ("max_position", c_int32),
                 ("loop_start", c_int32), ("loop_stop", c_int32), ("loop_times", c_int32), ("norm_eps", c_float), ("residual_mult", c_float), ("logit_softcap", c_float),
-                ("gemm_variant", c_int32), ("reserved", c_int32 * 8)]
+                ("gemm_variant", c_int32), ("tied_head", c_int32), ("loop_mix", c_int32), ("bigram_buckets", c_int32), ("bigram_mul_prev", c_int64), ("bigram_mul_cur", c_int64),
+                ("reserved", c_int32 * 8)]
 
 
 def _load():
@@ -73,6 +77,8 @@ _SIGS = {
     "lmx_create_stack": (c_int32, [POINTER(LmxStackConfig), POINTER(LmxLayerConfig), POINTER(c_void_p)]),
     "lmx_stack_set_rope": (c_int32, [c_void_p, c_int32, c_int32, c_void_p, c_int32]),
     "lmx_row_pitch": (c_int32, [c_void_p]),
+    "lmx_input_pitch": (c_int32, [c_void_p]),
+    "lmx_recurrent": (c_int32, [c_void_p]),
     "lmx_vocab_pitch": (c_int32, [c_void_p]),
     "lmx_logit_dtype": (c_int32, [c_void_p]),
     "lmx_layer_runs": (c_int32, [c_void_p]),

@@ -14,6 +14,9 @@ def __getattr__(name):
     if name in ("SiteraxConfig", "SiteraxForCausalLM"):
         from . import siterax
         return getattr(siterax, name)
+    if name in ("VizosunConfig", "VizosunForCausalLM"):
+        from . import vizosun
+        return getattr(vizosun, name)
     if name == "load_model":
         from .registry import load_model
         return load_model

@@ -79,6 +79,7 @@ class EngineCausalLM:
     """A causal language model on one engine handle; see the module docstring for what a subclass provides."""
 
     tp_rank, tp_world = 0, 1
+    exact_prefixes = False              # sequences carry state that cannot be cut back (lmx_recurrent): a prefix is reused whole or not at all
 
     def _init_host_state(self) -> None:
         self.generation_config = None
@@ -526,10 +527,11 @@ class EngineCausalLM:
             if self._prefix is not None and embeds.shape[0] == 1 and (valid is None or bool(valid.all())):
                 keys = self._request_row_keys(ids, embeds.shape[1])
             if keys is not None:
-                holder, n_common = self._prefix.take(keys)
+                holder, n_common = self._prefix.take(keys, whole=self.exact_prefixes)
                 if holder is not None:
                     p = min(n_common, embeds.shape[1] - 1)        # at least one row goes through the decoder: its logits pick the first token
-                    p -= p % 8                                     # the fused q|k|v epilogue wants pos0 % 8 == 0
+                    if not self.exact_prefixes:
+                        p -= p % 8                                 # the fused q|k|v epilogue wants pos0 % 8 == 0
                     if p >= self._prefix.min_rows and lib.lmx_seq_truncate(holder.seqs[0], p, stream_handle()) == 0:
                         cache, reused = holder, p
                         self._prefix.rows_reused += p
@@ -580,7 +582,7 @@ class EngineCausalLM:
             gen = np.asarray(list(out or [])[:-1], dtype=np.int64)
             full = np.concatenate([keys, gen]) if len(gen) else keys
             n = min(len(full), int(lib.lmx_seq_length(cache.seqs[0])))
-            if n < pc.min_rows:
+            if n < pc.min_rows or (self.exact_prefixes and n != int(lib.lmx_seq_length(cache.seqs[0]))):
                 cache.close()
                 return
             cache.row_keys = None

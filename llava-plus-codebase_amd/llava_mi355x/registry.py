@@ -38,6 +38,17 @@ def iter_checkpoint(path: str) -> Iterator[Tuple[str, torch.Tensor]]:
                 yield k, v
 
 
+def checkpoint_shapes(path: str) -> Dict[str, Tuple[int, ...]]:
+    """{key: shape} of a directory's *.safetensors, from their headers alone."""
+    from safetensors import safe_open
+    out: Dict[str, Tuple[int, ...]] = {}
+    for f in sorted(glob.glob(os.path.join(path, "*.safetensors"))):
+        with safe_open(f, framework="pt", device="cpu") as sf:
+            for k in sf.keys():
+                out[k] = tuple(sf.get_slice(k).get_shape())
+    return out
+
+
 @dataclass(frozen=True)
 class ModelFamily:
     name: str
@@ -62,6 +73,7 @@ def register(family: ModelFamily, *keys: str) -> None:
 
 register(ModelFamily("llava", "builder", "from_pretrained", multimodal=True), "llava", "LlavaLlamaForCausalLM")
 register(ModelFamily("siterax", "siterax", "SiteraxForCausalLM.from_pretrained"), "siterax", "SiteraxForCausalLM")
+register(ModelFamily("vizosun", "vizosun", "VizosunForCausalLM.from_pretrained"), "vizosun", "VizosunForCausalLM")
 
 
 def family_of(path: str) -> ModelFamily:
