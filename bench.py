@@ -61,11 +61,12 @@ def parse():
     ap.add_argument("--train-keep-gb", type=float, default=-1.0, help="config5: bytes of layer activations kept instead of recomputed (GB; < 0 = what 88 %% of the device "
                                                                       "memory leaves after a fully recomputing step, 0 = recompute every layer as the reference's gradient_checkpointing)")
     ap.add_argument("--train-seq", type=int, default=1024, help="config5: positions per sample after the image splice (the reference caps at 2048)")
-    ap.add_argument("--workload", default="config2", choices=["config2", "config3", "config5", "siterax"],
+    ap.add_argument("--workload", default="config2", choices=["config2", "config3", "config5", "siterax", "vizosun"],
                     help="config2 (default, BASELINE metric): one request, batch 1.  config3: LLaVA-1.5-13B geometry, 8 requests (8 images), "
                          "chunked prefill (512 rows), the 8 sequences decode together; prefill and decode reported separately.  config5: one "
                          "visual-instruction-tuning step (forward, backward, AdamW, ZeRO-2 over the ranks) of LLaVA-1.5-7B geometry.  siterax: prefill and decode of "
-                         "the Siterax decoder at real layer sizes beside the LLaMA decoder at equal size, with per-kernel roofline fractions (one GPU)")
+                         "the Siterax decoder at real layer sizes beside the LLaMA decoder at equal size, with per-kernel roofline fractions (one GPU).  vizosun: the same of the "
+                         "Vizosun decoder beside Siterax")
     ap.add_argument("--no-parity-probe", action="store_true", help="skip the live parity probe (the fp32 verification engine on the same bf16-rounded weights: "
                                                                   "last-position prefill logits and the first greedy ids of the timed request)")
     ap.add_argument("--no-pmc", action="store_true", help="skip the rocprofv3 --pmc passes that measure roofline.traffic")
@@ -937,6 +938,126 @@ def run_siterax(a, dev):
                       "rows": rows}), flush=True)
 
 
+# ---- Vizosun beside Siterax -------------------------------------------------------------------------------------------------------------------
+# name -> width, heads, head width, query latent, key / value latent, dense ff, (experts, active, expert ff), layers, vocab, window; the active feed-forward width of a
+# mixture equals the dense one.  Every fourth layer is latent attention, every second feed-forward a mixture.
+VIZOSUN_SIZES = {
+    "w2048": (2048, 16, 128, 768, 512, 5632, (16, 4, 1408), 12, 32000, 1024),
+    "w4096": (4096, 32, 128, 1536, 512, 11008, (16, 4, 2752), 12, 32000, 1024),
+}
+VIZOSUN_RANK = 128                   # inner size of the decay and output-gate projections
+PEAK_FP32_TFLOPS = 157.3             # vector fp32: what a recurrence kept in 32 bits is priced against
+
+
+def _vizosun_model(size, dev, dtype, max_position):
+    from llava_mi355x.vizosun import VizosunConfig, VizosunForCausalLM
+    W, H, D, Q, R, F, (E, top, EF), L, V, win = size
+    layers, shapes, A = [], [("embed", (V, W)), ("bigram", (8192, W)), ("final.norm", (W,))], VIZOSUN_RANK
+    for i in range(L):
+        p, lat, mix = f"l{i}.", i % 4 == 3, i % 2 == 1
+        layers.append({"type": "latent_attention" if lat else "channel_delta",
+                       "mixer": {"heads": H, "dim": D, "vdim": D, "q_rank": Q, "kv_rank": R, "scale": D ** -0.5, "mask": {"size": win}} if lat
+                       else {"heads": H, "kv_heads": H, "dim": D, "vdim": D, "conv": 4},
+                       "mlp": {"kind": "moe", "expert": {"ff": EF}, "router": {"experts": E, "top": top}} if mix else {"kind": "dense", "ff": F}})
+        shapes.append((p + "norm1", (W,)))
+        if lat:
+            shapes += [(p + "mix." + n, s) for n, s in (("dq", (Q, W)), ("dq.norm", (Q,)), ("uq", (H * D, Q)), ("dkv", (R, W)), ("dkv.norm", (R,)), ("uk", (H * D, R)), ("uv", (H * D, R)))]
+        else:
+            shapes += [(p + "mix." + n, (H * D, W)) for n in "qkv"] + [(p + f"mix.{n}.conv", (H * D, 4)) for n in "qkv"]
+            shapes += [(p + "mix." + n, s) for n, s in (("b", (H, W)), ("A_log", (H,)), ("dt_bias", (H * D,)), ("norm", (D,)), ("a1", (A, W)), ("a2", (H * D, A)), ("g1", (A, W)), ("g2", (H * D, A)))]
+        shapes.append((p + "mix.o", (W, H * D)))
+        if mix:
+            shapes += [(p + "mlp.router", (E, W)), (p + "mlp.router.b", (E,))]
+            shapes += [(p + f"mlp.e{e}.{n}", (W, EF) if n == "down" else (EF, W)) for e in range(E) for n in ("gate", "up", "down")]
+        else:
+            shapes += [(p + "mlp.gate", (F, W)), (p + "mlp.up", (F, W)), (p + "mlp.down", (W, F))]
+    c = VizosunConfig.from_dict({"vocab": V, "width": W, "layers": layers, "norm": {"eps": 1e-5}, "embedding": {"bigram": {"buckets": 8191, "mul_prev": 31, "mul_cur": 17}}, "loop": None}, dict(shapes))
+    return _random_weights(VizosunForCausalLM(c, dtype=dtype, device=dev, max_position=max_position), shapes, dev, dtype)
+
+
+def _vizosun_floors(size, T, ctx, n_batch, dec_steps, batch_steps):
+    """Roofline time of everything a kernel group does in the profiled passes (one prefill of T rows, dec_steps single and batch_steps batched steps)."""
+    W, H, D, Q, R, F, (E, top, EF), L, V, win = size
+    A, hd = VIZOSUN_RANK, H * D
+    hbm = lambda by: by / (PEAK_HBM_GBS * 1e9)
+    lin = lambda M, N, K, W_rows=None: max(2.0 * M * N * K / (PEAK_BF16_TFLOPS * 1e12), hbm(2.0 * ((W_rows or N) * K + M * K + M * N)))
+    seen = sum(min(i + 1, win) for i in range(T))
+    f = {}
+
+    def add(name, t):
+        f[name] = f.get(name, 0.0) + t
+    add("prefill.embed", hbm(8.0 * T * W))
+    for i in range(L):
+        lat, mix = i % 4 == 3, i % 2 == 1
+        n_in = Q + R if lat else 3 * hd + H + 2 * A
+        add("prefill.gemm.qkv", lin(T, n_in, W))
+        add("decode.gemv.qkv", hbm(2.0 * n_in * W) * dec_steps)
+        if lat:
+            add("prefill.latent_norm", hbm(4.0 * T * (Q + R)))
+            add("prefill.gemm.uq", lin(T, hd, Q)); add("prefill.gemm.ukv", lin(T, 2 * hd, R)); add("prefill.kv_rows", hbm(8.0 * T * hd))
+            add("prefill.attn", 4.0 * seen * hd / (PEAK_BF16_TFLOPS * 1e12))
+            for pre, n, ctx_, steps in (("decode", 1, ctx, dec_steps), ("decode_batch", n_batch, ctx // 2, batch_steps)):
+                if pre == "decode":
+                    add("decode.gemv.uq", hbm(2.0 * hd * Q) * steps)
+                add(pre + ".latent_q", hbm(2.0 * hd * R) * steps); add(pre + ".latent_o", hbm(2.0 * hd * R) * steps)
+                add(pre + ".attn", hbm(2.0 * min(ctx_, win) * R * n) * steps)
+        else:
+            add("prefill.gemm.decay_gate", lin(T, 2 * hd, A))
+            add("prefill.delta.prep", hbm(T * hd * (2.0 * 4 + 4 + 4 + 4 + 2)))
+            add("prefill.delta.scan", max(hbm(T * hd * (12.0 + 2 + 4)), 7.0 * T * hd * D / (PEAK_FP32_TFLOPS * 1e12)))
+            add("prefill.delta.gate", hbm(T * hd * 8.0))
+            for pre, n, steps in (("decode", 1, dec_steps), ("decode_batch", n_batch, batch_steps)):
+                add(pre + ".delta", hbm(8.0 * hd * D * n + 4.0 * hd * A) * steps)
+        add("prefill.gemm.o", lin(T, W, hd + (0 if mix else F)))
+        add("decode.gemv.o", hbm(2.0 * W * (hd + (0 if mix else F))) * dec_steps)
+        add("prefill.residual_norm", hbm(12.0 * T * W + (2.0 * top * T * W if mix else 0)))
+        if mix:
+            add("prefill.moe.router", hbm(2.0 * T * W)); add("prefill.moe.gate_up", lin(T * top, 2 * EF, W, 2 * EF * E)); add("prefill.moe.down", lin(T * top, W, EF, W * E))
+            for pre, n, steps in (("decode", 1, dec_steps), ("decode_batch", n_batch, batch_steps)):
+                hit = min(E, n * top)
+                add(pre + ".moe.router", hbm(2.0 * E * W) * steps)
+                add(pre + ".moe.gate_up", hbm(4.0 * EF * W * hit) * steps); add(pre + ".moe.down", hbm(2.0 * EF * W * hit) * steps)
+        else:
+            add("prefill.gemm.gate_up", lin(T, 2 * F, W))
+            add("decode.gemv.gate_up", hbm(4.0 * W * F) * dec_steps)
+    add("prefill.residual_norm", hbm(6.0 * T * W))
+    add("decode.gemv.lm_head", hbm(2.0 * V * W) * dec_steps)
+    return f
+
+
+def run_vizosun(a, dev):
+    dtype = {"bf16": torch.bfloat16, "f16": torch.float16}[a.dtype]
+    T, ctx, new = 2048, 2048, 64
+    rows, first = {}, None
+    for name, size in VIZOSUN_SIZES.items():
+        W, H, D, Q, R, F, _, L, V, win = size
+        res = {}
+        for kind in ("vizosun", "siterax"):
+            sx = (W, H, max(1, H // 4), D, F, L, V, win)
+            model = _vizosun_model(size, dev, dtype, 4096) if kind == "vizosun" else _siterax_model(sx, dev, dtype, 4096)
+            fig, prof, bprof = _time_decoder(model, T, ctx, new, a.steps, a.warmup)
+            if kind == "vizosun":
+                floors = _vizosun_floors(size, T, ctx, 32, 8, 4)
+                fig["kernels"] = {k: {"us": round(ms * 1e3 / max(1, n), 2), "launches": n, "total_us": round(ms * 1e3, 1), **({"roofline_frac": round(floors[k] * 1e3 / ms, 3)} if k in floors and ms > 0 else {})}
+                                  for k, (ms, n) in sorted({**prof, **bprof}.items())}
+            else:
+                fig["kernels"] = _kernel_rooflines(prof, sx, (H, max(1, H // 4), D), T, ctx, 1)
+                fig["kernels"].update(_kernel_rooflines(bprof, sx, (H, max(1, H // 4), D), T, ctx // 2, 32))
+            res[kind] = fig
+            del model
+            torch.cuda.empty_cache()
+        for k in ("prefill", "decode", "decode_batch8", "decode_batch32"):
+            res[k + "_ratio"] = round(res["vizosun"][k + "_tok_s"] / res["siterax"][k + "_tok_s"], 3)
+        rows[name] = res
+        first = first or res
+        print(f"# {name}: prefill {res['prefill_ratio']} x, decode {res['decode_ratio']} x, batch 32 {res['decode_batch32_ratio']} x Siterax", file=sys.stderr, flush=True)
+    print(json.dumps({"metric": "vizosun_decode_tokens_per_s", "value": first["vizosun"]["decode_tok_s"], "unit": "tok/s", "n_gpus": 1, "steps": a.steps, "warmup": a.warmup,
+                      "ms_per_step": first["vizosun"]["decode_ms"], "higher_is_better": True, "scaling": "weak", "vs_baseline": None, "dtype": a.dtype, "data": "synthetic (random weights)",
+                      "config": {"workload": f"vizosun: prefill of {T} rows, {new} greedy tokens at context {ctx}, decode batches of 8 and 32 at context {ctx // 2}",
+                                 "sizes": {k: dict(zip(("width", "heads", "dim", "q_rank", "kv_rank", "ff", "experts_active_ff", "layers", "vocab", "window"), v)) for k, v in VIZOSUN_SIZES.items()}},
+                      "rows": rows}), flush=True)
+
+
 def main():
     a = parse()
     world = int(os.environ.get("WORLD_SIZE", "1"))
@@ -959,6 +1080,9 @@ def main():
         else:
             dist.init_process_group("nccl", device_id=dev)
 
+    if a.workload == "vizosun":
+        run_vizosun(a, dev)
+        return
     if a.workload == "siterax":
         run_siterax(a, dev)
         return
