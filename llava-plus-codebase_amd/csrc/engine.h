@@ -71,7 +71,7 @@ struct StackLayer {
 // one execution of a layer: own slice of the K and V^T caches (byte offsets; a latent layer's rows are in the K cache) and of the recurrent state (state, ring).
 // inject: the embedding row is added first; mix: a pass of the loop begins (x <- W [x; embedding row])
 struct StackRun { int layer; bool inject, mix; size_t k_off, v_off, s_off, r_off; };
-struct StackWs { void *q, *qlat, *olat, *act, *slots, *cat; int* ids; float* wt; };      // activations beside the ones every decoder has
+struct StackWs { void *q, *qlat, *olat, *act, *slots, *cat, *plan; int* ids; float* wt; };      // activations beside the ones every decoder has
 struct Stack {
     lmx_stack_config c{};
     std::vector<StackLayer> layers;
@@ -86,6 +86,8 @@ struct Stack {
     std::vector<float*> rope; std::vector<int> rope_dims;
     ~Stack() { for (float* p : rope) if (p) (void)hipFree(p); }
 };
+struct StackProf;                                        // profile names of a kind of step (stack_mixers.cpp)
+extern const StackProf stack_prof_prefill, stack_prof_decode, stack_prof_batch;
 struct StackOutputs {
     float* logits = nullptr;                             // rows [wanted][V] in the order of the sequences and of `want`
     const std::vector<int>* want = nullptr;              // per sequence: wanted rows, ascending (null: every row)
@@ -205,10 +207,10 @@ struct Model {
     // a mixer over the normed rows x of a piece -> rows [an] of pitch out_k; qkv: its projection rows
     void stack_mix_prefill(int r, Seq* const* seqs, const std::vector<Segment>& seg, int fill, const void* x, void* qkv, void* mix, void* scratch, void* skw, hipStream_t st);
     size_t stack_mix_scratch(int rows, int keys) const;
-    void stack_moe_prefill(const StackLayer& l, const void* x, int rows, const StackWs& w, hipStream_t st);
     // the same over one new token of every sequence (tab: batch; else `one`), projection rows already there
     void stack_mix_decode(int r, const DecodeFusedSeq* tab, const DecodeFusedSeq& one, int n, int max_len, void* qkv, void* mix, const StackWs& w, Batch* b, hipStream_t st);
-    void stack_moe_decode(const StackLayer& l, const void* x, int n, const StackWs& w, bool batch, hipStream_t st);
+    void stack_moe(const StackLayer& l, const void* x, int rows, const StackWs& w, const StackProf& pn, hipStream_t st);
+    void stack_heads(const GroupGemvArgs& g, int n, hipStream_t st);
     // ---- options a caller may flip on a live model (lmx_model_set_option; defaults from the environment at creation) ----------------------------------
     // fuse_rope: RoPE + KV append in the prefill's q|k|v GEMM epilogue (gemm8p.hip qkv_rope_epilogue) instead of a rope_kv launch — bit-identical, faster
     // vis_pack:  CLIP K / V^T pack in the tower's q|k|v GEMM epilogue instead of a pack launch — bit-identical, launch count

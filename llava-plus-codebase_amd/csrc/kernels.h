@@ -221,19 +221,20 @@ struct DeltaShape {
 };
 struct DeltaWeights { const void* conv; const void* A_log; const void* dt_bias; const void* norm; };      // conv [taps][channels], A_log [H], dt_bias [H][DK], norm [DV]
 constexpr int DELTA_MAX_SEG = 16;
-struct DeltaSeg { int row0, n, pos0; float* state; void* ring; };        // rows [row0, row0 + n) of the piece continue a sequence at position pos0 (0: from a zero state)
+struct DeltaSeg { int row0, n, pos0, chunk0; float* state; void* ring; };        // chunk0: chunks (16 tokens) of the segments ahead of it.  Rows [row0, row0 + n) of the piece continue a sequence at position pos0 (0: from a zero state)
 struct DeltaPrefillArgs {
     DeltaShape s; DeltaWeights w;
     const void* proj; int ld;            // projection rows
     const void* ag; int ag_ld;           // decay pre-activations [H][DK] | output gates [H][DV]
-    float* qk; float* g; void* v; float* sc; float* o;      // scratch rows: [G][2][DK] unit q, k | [H][DK] decays | [H][DV] | [H] {beta, q . k} pairs | [H][DV]
+    // scratch per (chunk, head) — decayed k and q [16][DK], written-out keys [DK][16], the chunk's decay [DK], T and P [16][16], values [DV][16] — and read-outs per row [H][DV]
+    float *kd, *qd, *kt, *dc, *tm, *pm; void* v; float* o;
     void* out; int out_ld;               // [H][DV] rows
     float eps;
     int n_seg; DeltaSeg seg[DELTA_MAX_SEG];
 };
 size_t delta_scratch_bytes(const DeltaShape& s, int rows, int es);
 void delta_carve(DeltaPrefillArgs& a, void* scratch, int rows, int es);
-void launch_delta_prep(int dtype, const DeltaPrefillArgs& a, hipStream_t st);      // convolutions, unit norms, decays, step sizes
+void launch_delta_prep(int dtype, const DeltaPrefillArgs& a, hipStream_t st);      // convolutions, unit norms, decays, step sizes, the chunks' matrices
 void launch_delta_scan(int dtype, const DeltaPrefillArgs& a, hipStream_t st);      // the recurrence; leaves state and ring behind
 void launch_delta_gate(int dtype, const DeltaPrefillArgs& a, hipStream_t st);      // root-mean-square norm and output gate
 struct DeltaDecodeArgs {                 // one new token per sequence, everything in one launch
@@ -273,6 +274,23 @@ struct GroupGemvArgs {                   // slot = blockIdx.y.  ids: group = ids
     const int* ids = nullptr; int per_row = 1, groups = 1;
 };
 void launch_group_gemv(int dtype, const GroupGemvArgs& a, int slots, hipStream_t st);
+// many rows per group: MFMA tiles.  With a plan (mixtures) tile rows are slots: x row slot / per_row, c row slot; without one every group takes rows [0, rows)
+constexpr int GROUP_MIN_BM = 32;
+struct GroupTile { int group, row0, rows, first, n_tiles; int pad[3]; };      // rows [row0, row0 + rows) of `order`; the group's first tile and tile count
+struct GroupPlan { int* order = nullptr; GroupTile* tiles = nullptr; int* n_tiles = nullptr; };
+size_t group_plan_bytes(int slots);
+GroupPlan group_plan_at(void* base, int slots);
+int group_gemm_bm(int slots, int groups);                        // rows of a tile
+bool group_gemm_applies(int dtype, int slots, int groups);
+void launch_group_plan(const int* ids, int slots, int groups, int bm, const GroupPlan& p, hipStream_t st);
+struct GroupGemmArgs {
+    const void* X; const void* W; void* C;
+    int N, K, ldx, ldw, ldc; size_t w_group;
+    int rows, groups;                    // rows: with a plan all slots, else those of one group
+    int x_group = 0, c_group = 0, act = 0, per_row = 1;
+    GroupPlan plan{};
+};
+void launch_group_gemm(int dtype, const GroupGemmArgs& a, int bm, hipStream_t st);
 struct MoeRouterArgs { const void* x; const void* w; const void* bias; int ldx, K, E, top; int* ids; float* wt; };      // ids / wt [rows][top]: the largest logits and their softmax
 void launch_moe_router(int dtype, const MoeRouterArgs& a, int rows, hipStream_t st);
 

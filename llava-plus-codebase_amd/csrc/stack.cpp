@@ -479,7 +479,7 @@ void Model::stack_prefill(Seq* const* seqs, const void* const* embeds, const int
                 } else yy = nullptr;
             }
             const int top = l.moe() ? d.top_experts : 0;
-            if (top) stack_moe_prefill(l, x, fill, sw, st);
+            if (top) stack_moe(l, x, fill, sw, stack_prof_prefill, st);
             const StackStep sp = stack_step(S, r, l.ff && !l.parallel() ? 1 : 0, final_norm);
             if (out.hidden) {
                 // residual trace: the stream right after this run, before anything the next run adds
@@ -635,7 +635,7 @@ void Model::stack_decode_step(Seq* s, hipStream_t st, int64_t* id_out) {
                 plain("decode.gemv.down", s->d_act, l.wd, s->d_y, H, l.ff);
             } else { residual(sp, y, 0, false); y = nullptr; }
         }
-        if (l.moe()) { stack_moe_decode(l, s->d_x, 1, s->sw, false, st); top = l.c.top_experts; }
+        if (l.moe()) { stack_moe(l, s->d_x, 1, s->sw, stack_prof_decode, st); top = l.c.top_experts; }
         before = stack_step(S, r, l.ff && !l.parallel() ? 1 : 0, final_norm);
     }
     {
@@ -703,7 +703,7 @@ void Model::stack_decode_batch_step(Batch* b, Seq* const* seqs, int n, int64_t* 
                 linear(GemmArgs{b->act, l.wd, b->y, nullptr, nullptr, n, H, l.ff, l.ff, l.ff, H, 0, kActNone}, l.sw_d);
             } else yy = nullptr;
         }
-        if (l.moe()) stack_moe_decode(l, b->x, n, b->sw, true, st);
+        if (l.moe()) stack_moe(l, b->x, n, b->sw, stack_prof_batch, st);
         norm(b->xr, yy, l.moe() ? l.c.top_experts : 0, stack_step(S, r, l.ff && !l.parallel() ? 1 : 0, final_norm));
     }
     GemmArgs ga{b->x, lm_head, b->logits, nullptr, nullptr, n, V, H, H, H, V, 0, kActNone};

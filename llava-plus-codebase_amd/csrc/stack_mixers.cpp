@@ -4,13 +4,18 @@
 
 namespace lmx {
 
+struct StackProf { const char *delta, *norm, *uq, *qlat, *attn, *olat, *router, *plan, *gate_up, *down; };
+#define NAMES(P, UQ) {P ".delta", P ".latent_norm", UQ, P ".latent_q", P ".attn", P ".latent_o", P ".moe.router", P ".moe.plan", P ".moe.gate_up", P ".moe.down"}
+const StackProf stack_prof_prefill = NAMES("prefill", "prefill.gemm.uq"), stack_prof_decode = NAMES("decode", "decode.gemv.uq"), stack_prof_batch = NAMES("decode_batch", "decode_batch.linear");
+#undef NAMES
+
 static int round_up(int a, int b) { return (a + b - 1) / b * b; }
 static size_t up256(size_t b) { return (b + 255) / 256 * 256; }
 
 size_t Stack::ws_bytes(int rows, int H, int es, bool decode) const {
     const size_t r = (size_t)rows;
     return (decode ? up256(r * q_n * es) + 2 * up256(r * lat_n * es) : 0) + up256(r * moe_act * es) + up256(r * moe_top * H * es) + 2 * up256(r * moe_top * 4) +
-           (c.loop_mix ? up256(r * 2 * H * es) : 0);
+           (moe_top ? up256(group_plan_bytes(rows * moe_top)) : 0) + (c.loop_mix ? up256(r * 2 * H * es) : 0);
 }
 
 StackWs Stack::ws(void* base, int rows, int H, int es, bool decode) const {
@@ -23,6 +28,7 @@ StackWs Stack::ws(void* base, int rows, int H, int es, bool decode) const {
     w.slots = take(r * moe_top * H * es);
     w.ids = static_cast<int*>(take(r * moe_top * 4));
     w.wt = static_cast<float*>(take(r * moe_top * 4));
+    if (moe_top) w.plan = take(group_plan_bytes(rows * moe_top));
     if (c.loop_mix) w.cat = take(r * 2 * H * es);
     return w;
 }
@@ -68,10 +74,11 @@ void Model::stack_mix_prefill(int r, Seq* const* seqs, const std::vector<Segment
         a.out = mix; a.out_ld = l.out_k; a.eps = S.c.norm_eps;
         for (size_t s0 = 0; s0 < seg.size(); s0 += DELTA_MAX_SEG) {
             a.n_seg = (int)std::min(seg.size() - s0, (size_t)DELTA_MAX_SEG);
-            for (int i = 0; i < a.n_seg; ++i) {
+            for (int i = 0, chunks = 0; i < a.n_seg; ++i) {
                 const Segment& g = seg[s0 + (size_t)i];
                 char* rs = seqs[g.seq]->rs.as<char>();
-                a.seg[i] = DeltaSeg{g.dst0, g.n, g.pos0, reinterpret_cast<float*>(rs + run.s_off), rs + run.r_off};
+                a.seg[i] = DeltaSeg{g.dst0, g.n, g.pos0, chunks, reinterpret_cast<float*>(rs + run.s_off), rs + run.r_off};
+                chunks += (g.n + 15) / 16;
             }
             { LMX_PROF_K("prefill.delta.prep"); launch_delta_prep(dt, a, st); }
             { LMX_PROF_K("prefill.delta.scan"); launch_delta_scan(dt, a, st); }
@@ -110,34 +117,15 @@ void Model::stack_mix_prefill(int r, Seq* const* seqs, const std::vector<Segment
     }
 }
 
-void Model::stack_moe_prefill(const StackLayer& l, const void* x, int rows, const StackWs& w, hipStream_t st) {
-    const int dt = cfg.dtype, top = l.c.top_experts;
-    { LMX_PROF_K("prefill.moe.router"); launch_moe_router(dt, MoeRouterArgs{x, l.wr, l.br, H, H, l.c.experts, top, w.ids, w.wt}, rows, st); }
-    GroupGemvArgs g{x, l.wgu, w.act, 2 * l.ff, H, H, H, l.ff, (size_t)2 * l.ff * H};
-    g.act = l.act(); g.ids = w.ids; g.per_row = top;
-    { LMX_PROF_K("prefill.moe.gate_up"); launch_group_gemv(dt, g, rows * top, st); }
-    GroupGemvArgs o{w.act, l.wd, w.slots, H, l.ff, l.ff, l.ff, H, (size_t)H * l.ff};
-    o.ids = w.ids;
-    { LMX_PROF_K("prefill.moe.down"); launch_group_gemv(dt, o, rows * top, st); }
-}
-
 // ---------------------------------------------------------------------------------------------------------------
 // one new token per sequence
 // ---------------------------------------------------------------------------------------------------------------
-struct ProfNames { const char *delta, *norm, *uq, *qlat, *attn, *olat, *router, *gate_up, *down; };
-static const ProfNames& prof_names(bool batch) {
-    static const ProfNames one{"decode.delta", "decode.latent_norm", "decode.gemv.uq", "decode.latent_q", "decode.attn", "decode.latent_o", "decode.moe.router", "decode.moe.gate_up", "decode.moe.down"};
-    static const ProfNames many{"decode_batch.delta", "decode_batch.latent_norm", "decode_batch.linear", "decode_batch.latent_q", "decode_batch.attn", "decode_batch.latent_o", "decode_batch.moe.router",
-                                "decode_batch.moe.gate_up", "decode_batch.moe.down"};
-    return batch ? many : one;
-}
-
 void Model::stack_mix_decode(int r, const DecodeFusedSeq* tab, const DecodeFusedSeq& one, int n, int max_len, void* qkv, void* mix, const StackWs& w, Batch* b, hipStream_t st) {
     Stack& S = *stk;
     const StackLayer& l = S.layers[(size_t)S.runs[(size_t)r].layer];
     const lmx_layer_config& d = l.c;
     const int dt = cfg.dtype;
-    const ProfNames& pn = prof_names(b != nullptr);
+    const StackProf& pn = b ? stack_prof_batch : stack_prof_decode;
     if (d.mixer == LMX_MIXER_DELTA) {
         DeltaDecodeArgs a{};
         a.s = l.ds; a.w = DeltaWeights{l.conv, l.a_log, l.dt_bias, l.onorm};
@@ -162,7 +150,7 @@ void Model::stack_mix_decode(int r, const DecodeFusedSeq* tab, const DecodeFused
     // q W_uk of every head: the scores against all cached latents are then plain dot products
     GroupGemvArgs g{w.q, l.wuk_t, w.qlat, l.R, l.D, l.an, l.D, d.n_heads * l.R, (size_t)l.R * l.D};
     g.groups = d.n_heads; g.x_group = l.D; g.c_group = l.R;
-    { LMX_PROF_K(pn.qlat); launch_group_gemv(dt, g, n * d.n_heads, st); }
+    { LMX_PROF_K(pn.qlat); stack_heads(g, n, st); }
     {
         LMX_PROF_K(pn.attn);
         LatentDecodeArgs a;
@@ -175,19 +163,42 @@ void Model::stack_mix_decode(int r, const DecodeFusedSeq* tab, const DecodeFused
     }
     GroupGemvArgs o{w.olat, static_cast<char*>(l.wukv) + (size_t)l.an * l.R * es, mix, l.D, l.R, d.n_heads * l.R, l.R, l.out_k, (size_t)l.D * l.R};
     o.groups = d.n_heads; o.x_group = l.R; o.c_group = l.D;
-    { LMX_PROF_K(pn.olat); launch_group_gemv(dt, o, n * d.n_heads, st); }
+    { LMX_PROF_K(pn.olat); stack_heads(o, n, st); }
 }
 
-void Model::stack_moe_decode(const StackLayer& l, const void* x, int n, const StackWs& w, bool batch, hipStream_t st) {
-    const int dt = cfg.dtype, top = l.c.top_experts;
-    const ProfNames& pn = prof_names(batch);
-    { LMX_PROF_K(pn.router); launch_moe_router(dt, MoeRouterArgs{x, l.wr, l.br, H, H, l.c.experts, top, w.ids, w.wt}, n, st); }
+// every head's rows through the head's own weight
+void Model::stack_heads(const GroupGemvArgs& g, int n, hipStream_t st) {
+    const int dt = cfg.dtype;
+    if (dt == kF32 || n < 4) { launch_group_gemv(dt, g, n * g.groups, st); return; }
+    GroupGemmArgs a{g.X, g.W, g.C, g.N, g.K, g.ldx, g.ldw, g.ldc, g.w_group, n, g.groups};
+    a.x_group = g.x_group; a.c_group = g.c_group;
+    launch_group_gemm(dt, a, n <= 32 ? 32 : 64, st);
+}
+
+// ---------------------------------------------------------------------------------------------------------------
+// mixture of experts: choices, then both products with the rows as they are (few: weights streamed per row) or sorted by expert (MFMA tiles)
+// ---------------------------------------------------------------------------------------------------------------
+void Model::stack_moe(const StackLayer& l, const void* x, int rows, const StackWs& w, const StackProf& pn, hipStream_t st) {
+    const int dt = cfg.dtype, top = l.c.top_experts, E = l.c.experts, slots = rows * top;
+    { LMX_PROF_K(pn.router); launch_moe_router(dt, MoeRouterArgs{x, l.wr, l.br, H, H, E, top, w.ids, w.wt}, rows, st); }
+    if (group_gemm_applies(dt, slots, E)) {
+        const int bm = group_gemm_bm(slots, E);
+        const GroupPlan plan = group_plan_at(w.plan, slots);
+        { LMX_PROF_K(pn.plan); launch_group_plan(w.ids, slots, E, bm, plan, st); }
+        GroupGemmArgs g{x, l.wgu, w.act, 2 * l.ff, H, H, H, l.ff, (size_t)2 * l.ff * H, slots, E};
+        g.act = l.act(); g.per_row = top; g.plan = plan;
+        { LMX_PROF_K(pn.gate_up); launch_group_gemm(dt, g, bm, st); }
+        GroupGemmArgs o{w.act, l.wd, w.slots, H, l.ff, l.ff, l.ff, H, (size_t)H * l.ff, slots, E};
+        o.plan = plan;
+        { LMX_PROF_K(pn.down); launch_group_gemm(dt, o, bm, st); }
+        return;
+    }
     GroupGemvArgs g{x, l.wgu, w.act, 2 * l.ff, H, H, H, l.ff, (size_t)2 * l.ff * H};
     g.act = l.act(); g.ids = w.ids; g.per_row = top;
-    { LMX_PROF_K(pn.gate_up); launch_group_gemv(dt, g, n * top, st); }
+    { LMX_PROF_K(pn.gate_up); launch_group_gemv(dt, g, slots, st); }
     GroupGemvArgs o{w.act, l.wd, w.slots, H, l.ff, l.ff, l.ff, H, (size_t)H * l.ff};
     o.ids = w.ids;
-    { LMX_PROF_K(pn.down); launch_group_gemv(dt, o, n * top, st); }
+    { LMX_PROF_K(pn.down); launch_group_gemv(dt, o, slots, st); }
 }
 
 }  // namespace lmx
