@@ -45,13 +45,11 @@ __device__ __forceinline__ float silu_acc(float z) { return z / (1.f + expf(-z))
 // ---------------------------------------------------------------------------------------------------------------
 constexpr int DELTA_C = 16;              // tokens of a chunk
 
-__device__ __forceinline__ const DeltaSeg* delta_segment(const DeltaPrefillArgs& a, int tile, int& t0) {
-    for (int s = 0; s < a.n_seg; ++s) {
-        const int nt = (a.seg[s].n + DELTA_C - 1) / DELTA_C;
-        if (tile < nt) { t0 = tile * DELTA_C; return &a.seg[s]; }
-        tile -= nt;
-    }
-    return nullptr;
+// segment of a chunk (its index, or -1)
+__device__ __forceinline__ int delta_segment(const DeltaPrefillArgs& a, int chunk) {
+    int s = a.n_seg - 1;
+    while (s > 0 && a.seg[s].chunk0 > chunk) --s;
+    return (chunk - a.seg[s].chunk0) * DELTA_C < a.seg[s].n ? s : -1;
 }
 
 // 8 channels of token t: sum over the taps, then silu.  Inputs before the portion come from the ring, before the sequence they are zero
@@ -63,11 +61,14 @@ __device__ __forceinline__ void conv_silu8(const DeltaPrefillArgs& a, const Delt
     const T* ring = reinterpret_cast<const T*>(sg.ring) + c;
 #pragma unroll
     for (int e = 0; e < 8; ++e) out[e] = 0.f;
+#pragma unroll 4
     for (int j = 0; j < taps; ++j) {
         const int r = t - (taps - 1) + j, p = sg.pos0 + r;
         if (p < 0) continue;
         float x[8], f[8];
-        load8<T>(r >= 0 ? proj + (size_t)r * a.ld : ring + (size_t)(p % taps) * C, x);
+        const T* src = proj + (ptrdiff_t)r * a.ld;
+        if (r < 0) src = ring + (size_t)(p % taps) * C;
+        load8<T>(src, x);
         load8<T>(w + (size_t)j * C, f);
 #pragma unroll
         for (int e = 0; e < 8; ++e) out[e] = fmaf(x[e], f[e], out[e]);
@@ -84,10 +85,10 @@ __global__ __launch_bounds__(256) void delta_prep_kernel(DeltaPrefillArgs a) {
     float *g = dsm, *k = g + C * DK, *q = k + C * DK;        // [C][DK]; the value tile comes first in the same place, the written-out keys last
     __shared__ float A[C][C], P[C][C], beta[C];
     const int tid = threadIdx.x, H = a.s.H, G = a.s.G, DV = a.s.DV;
-    int t0 = 0;
-    const DeltaSeg* sp = delta_segment(a, blockIdx.x, t0);
-    if (!sp) return;
-    const DeltaSeg sg = *sp;
+    const int si = __builtin_amdgcn_readfirstlane(delta_segment(a, blockIdx.x));
+    if (si < 0) return;
+    const DeltaSeg sg = a.seg[si];
+    const int t0 = ((int)blockIdx.x - sg.chunk0) * DELTA_C;
     const int nt = sg.n - t0 < C ? sg.n - t0 : C;
     const int h = blockIdx.y, kh = h / (H / G);
     const size_t ch = (size_t)(sg.chunk0 + t0 / C) * H + h;
@@ -204,7 +205,7 @@ __device__ __forceinline__ f32x4 ldg4(const float* p) { return *reinterpret_cast
 // lanes: register i of lane l of an accumulator is row 4 (l / 16) + i, column l % 16, which as a B operand is k index l / 16 of the i-th of four products whose A operands
 // hold columns 4 (l / 16) + i.  The waves' parts of (D k) S and of o meet in LDS.
 template <typename T, int LPC>
-__global__ __launch_bounds__(256) void delta_scan_kernel(DeltaPrefillArgs a) {
+__global__ __launch_bounds__(256, 1) void delta_scan_kernel(DeltaPrefillArgs a) {
     constexpr int DK = LPC * 8, NT = DK / 64, C = DELTA_C;
     __shared__ __attribute__((aligned(16))) f32x4 wb[2][4][64], ob[2][4][64];
     const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
@@ -239,10 +240,7 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(DeltaPrefillArgs a) {
         if (n * C + t < sg.n) a.o[((size_t)sg.row0 + n * C + t) * H * DV + (size_t)h * DV + c0 + col] = v;
     };
     const int nc = (sg.n + C - 1) / C;
-    Chunk cur, nxt;
-    fetch(0, cur);
-    for (int n = 0; n < nc; ++n) {
-        if (n + 1 < nc) fetch(n + 1, nxt);
+    auto step = [&](int n, const Chunk& cur) {
         f32x4 W = {0.f, 0.f, 0.f, 0.f}, O = W, U = W, X;
 #pragma unroll
         for (int j = 0; j < NT; ++j)
@@ -253,7 +251,7 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(DeltaPrefillArgs a) {
         for (int j = 0; j < NT; ++j)
 #pragma unroll
             for (int i = 0; i < 4; ++i) O = mfma4(cur.qd[j][i], S[j][i], O);
-        // LDS only: a full barrier would also wait for the next chunk's loads
+        // LDS only: a full barrier would also wait for the chunks that are on their way
         asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
         __builtin_amdgcn_s_barrier();
         asm volatile("" ::: "memory");
@@ -274,8 +272,19 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(DeltaPrefillArgs a) {
         O = mfma4(cur.pm, wave == 0 ? U[0] : wave == 1 ? U[1] : wave == 2 ? U[2] : U[3], O);      // a quarter of P U per wave
         ob[n & 1][wave][lane] = O;
         if (n > 0) put_o(n - 1);
-        cur = nxt;
-    }
+    };
+    // NB chunks in registers, NB - 1 of them on their way; past the last chunk the last one is read again
+    constexpr int NB = NT >= 4 ? 3 : 4;
+    Chunk buf[NB];
+    auto at = [&](int n) { return n < nc ? n : nc - 1; };
+#pragma unroll
+    for (int u = 0; u < NB - 1; ++u) fetch(at(u), buf[u]);
+    int n = 0;
+    for (; n + NB <= nc; n += NB)
+#pragma unroll
+        for (int u = 0; u < NB; ++u) { fetch(at(n + u + NB - 1), buf[(u + NB - 1) % NB]); step(n + u, buf[u]); }
+#pragma unroll
+    for (int u = 0; u < NB - 1; ++u) if (n + u < nc) step(n + u, buf[u]);
     __syncthreads();
     put_o(nc - 1);
 #pragma unroll

@@ -61,7 +61,7 @@ void Model::stack_mix_prefill(int r, Seq* const* seqs, const std::vector<Segment
     const int dt = cfg.dtype, gv = cfg.gemm_variant;
     char* p = static_cast<char*>(scratch);
     auto take = [&](size_t bytes) -> char* { char* q = p; p += up256(bytes); return q; };
-    auto gemm = [&](const char* name, GemmArgs g) { LMX_PROF_K(name); g.skw = skw; launch_gemm(dt, g, gv, st); };
+    auto gemm = [&](const char* name, GemmArgs g) { LMX_PROF_K(name); g.skw = g.K >= 1024 ? skw : nullptr; launch_gemm(dt, g, gv, st); };
     if (d.mixer == LMX_MIXER_DELTA) {
         DeltaPrefillArgs a{};
         a.s = l.ds; a.w = DeltaWeights{l.conv, l.a_log, l.dt_bias, l.onorm};
