@@ -844,12 +844,12 @@ def _time_decoder(model, T, ctx, new_tokens, steps, warmup, batches=(8, 32)):
     from llava_mi355x._C import check, lib, ptr, stream_handle
     from llava_mi355x.batching import DecodeBatch
     from llava_mi355x.engine_lm import LmxKVCache
-    ids = torch.randint(0, model.config.vocab_size, (1, max(T, ctx)), device=model.device)
+    ids = torch.randint(0, model.config.vocab_size, (1, max(T, ctx) + 16 * max(batches)), device=model.device)
     emb = model.get_model().embed_tokens(ids)[0].contiguous()
 
-    def prefill(rows):
+    def prefill(rows, member=0):         # the members of a batch have different prompts
         c = LmxKVCache(model, 1)
-        check(lib.lmx_prefill(model._h, c.seqs[0], ptr(emb), rows, 0, None, 0, 1, stream_handle()), "lmx_prefill")
+        check(lib.lmx_prefill(model._h, c.seqs[0], ptr(emb[16 * member:]), rows, 0, None, 0, 1, stream_handle()), "lmx_prefill")
         return c
 
     def timed(fn):
@@ -870,7 +870,7 @@ def _time_decoder(model, T, ctx, new_tokens, steps, warmup, batches=(8, 32)):
     out = {"prefill_tok_s": round(T / statistics.median(pre), 1), "prefill_ms": round(statistics.median(pre) * 1e3, 3), "decode_tok_s": round(1 / statistics.median(dec), 1),
            "decode_ms": round(statistics.median(dec) * 1e3, 4)}
     for n in batches:
-        cs = [prefill(ctx // 2) for _ in range(n)]
+        cs = [prefill(ctx // 2, i) for i in range(n)]
         b = DecodeBatch(model, n)
         ts = []
         for it in range(warmup + steps):
@@ -894,7 +894,7 @@ def _time_decoder(model, T, ctx, new_tokens, steps, warmup, batches=(8, 32)):
         model.set_option("decode_splitq", 1)
     model.profile(False)
     n = batches[-1]
-    cs = [prefill(ctx // 2) for _ in range(n)]
+    cs = [prefill(ctx // 2, i) for i in range(n)]
     model.profile(True)
     b = DecodeBatch(model, n)
     b.step([x.seqs[0] for x in cs], None, 4, True, want_ids=False)
@@ -1014,7 +1014,7 @@ def _vizosun_floors(size, T, ctx, n_batch, dec_steps, batch_steps):
         if mix:
             add("prefill.moe.router", hbm(2.0 * T * W)); add("prefill.moe.gate_up", lin(T * top, 2 * EF, W, 2 * EF * E)); add("prefill.moe.down", lin(T * top, W, EF, W * E))
             for pre, n, steps in (("decode", 1, dec_steps), ("decode_batch", n_batch, batch_steps)):
-                hit = min(E, n * top)
+                hit = E * (1 - (1 - top / E) ** n)      # experts that n rows choose at random
                 add(pre + ".moe.router", hbm(2.0 * E * W) * steps)
                 add(pre + ".moe.gate_up", hbm(4.0 * EF * W * hit) * steps); add(pre + ".moe.down", hbm(2.0 * EF * W * hit) * steps)
         else:

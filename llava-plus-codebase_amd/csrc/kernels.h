@@ -264,6 +264,7 @@ struct LatentDecodeArgs {                // queries already in the latent space,
     float scale = 1.f;
 };
 void launch_latent_decode(int dtype, const LatentDecodeArgs& a, hipStream_t st);
+int latent_decode_split(int dtype, int R, int H, int n_seq, int span);      // n_split for a context of `span` keys
 
 // ---- grouped linears and mixtures of experts (moe.hip) -----------------------------------------------------------------------------------------------------------
 struct GroupGemvArgs {                   // slot = blockIdx.y.  ids: group = ids[slot], x row slot / per_row, c row slot.  no ids: group = slot % groups, x and c row slot / groups

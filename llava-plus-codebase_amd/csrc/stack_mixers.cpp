@@ -61,7 +61,11 @@ void Model::stack_mix_prefill(int r, Seq* const* seqs, const std::vector<Segment
     const int dt = cfg.dtype, gv = cfg.gemm_variant;
     char* p = static_cast<char*>(scratch);
     auto take = [&](size_t bytes) -> char* { char* q = p; p += up256(bytes); return q; };
-    auto gemm = [&](const char* name, GemmArgs g) { LMX_PROF_K(name); g.skw = g.K >= 1024 ? skw : nullptr; launch_gemm(dt, g, gv, st); };
+    auto gemm = [&](const char* name, GemmArgs g) { LMX_PROF_K(name);
+        // inner sizes of a few K-steps: the time is the launch's fixed part and the output; the smaller tiles write it sooner than the large ones
+        const int v = gv == 0 && dt != kF32 && g.K <= 512 ? (g.K <= 256 ? 5 : 18) : gv;
+        g.skw = g.K >= 1024 ? skw : nullptr;
+        launch_gemm(dt, g, v, st); };
     if (d.mixer == LMX_MIXER_DELTA) {
         DeltaPrefillArgs a{};
         a.s = l.ds; a.w = DeltaWeights{l.conv, l.a_log, l.dt_bias, l.onorm};
@@ -157,8 +161,7 @@ void Model::stack_mix_decode(int r, const DecodeFusedSeq* tab, const DecodeFused
         a.q = w.qlat; a.out = w.olat; a.tab = tab; a.one = one; a.n_seq = n; a.H = d.n_heads; a.R = l.R; a.s_max = s_max; a.window = d.window; a.scale = d.attn_scale;
         int span = max_len + 1;
         if (d.window > 0 && d.window < span) span = d.window;
-        const int chunks = std::max(1, std::min((span + 63) / 64, 32)), room = (1024 + d.n_heads * n - 1) / (d.n_heads * n);
-        a.n_split = std::max(1, std::min(chunks, room));
+        a.n_split = latent_decode_split(dt, l.R, d.n_heads, n, span);
         launch_latent_decode(dt, a, st);
     }
     GroupGemvArgs o{w.olat, static_cast<char*>(l.wukv) + (size_t)l.an * l.R * es, mix, l.D, l.R, d.n_heads * l.R, l.R, l.out_k, (size_t)l.D * l.R};

@@ -220,6 +220,23 @@ def test_a_far_token_stays_in_the_state(cuda, dt):
             assert rel((run(m, a, cuts) - run(m, b, cuts))[300:], (wa - wb)[300:]) < 2e-2
 
 
+@pytest.mark.parametrize("a_log,dt_bias", [(4.0, 4.0), (-9.0, -6.0), (1.0, 0.0)])
+def test_decays_of_any_strength(cuda, a_log, dt_bias):
+    """states that vanish within a token, that keep everything, and both next to each other in one head: prompts (in chunks), portions across their borders, decoding"""
+    cfg = config([delta(3, 1, 70, 40, 3, None), delta(2, 2, 64, 130, 4, dense(40))], 96, 80)
+    w = O.make_weights(cfg, 5, (33, 20))
+    for i in (0, 1):
+        w[f"l{i}.mix.A_log"] = torch.full_like(w[f"l{i}.mix.A_log"], a_log)
+        b = torch.full_like(w[f"l{i}.mix.dt_bias"], dt_bias)
+        b[::5] = -dt_bias
+        w[f"l{i}.mix.dt_bias"] = b
+    m, t = build_config(cfg, w, torch.float32), torch.randint(0, 80, (150,), generator=torch.Generator().manual_seed(3)).tolist()
+    want = O.logits(cfg, w, t)
+    for cuts in ((), (15, 16, 17, 31, 33, 64), (20,) + tuple(range(140, 150))):
+        got = run(m, t, cuts)
+        assert torch.isfinite(got).all() and rel(got, want) < TOL["f32"], cuts
+
+
 def test_the_first_tokens_of_a_sequence(cuda):
     """the row without a previous token, and convolutions that reach before the start; the second token looks back at the first, however it arrives"""
     for name in ("mixed", "odd", "wide"):

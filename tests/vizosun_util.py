@@ -38,10 +38,13 @@ CONFIGS = {
     "plain": config([latent(4, 48, 48, 40, 60, 0, dense(100)), delta(4, 4, 48, 30, 4, moe(56, 6, 4))], 120, 90, {"start": 0, "stop": 2, "times": 2}, bigram=None),
     # head vectors and latents past 128
     "wide": config([delta(2, 1, 150, 200, 4, dense(70)), latent(2, 160, 136, 200, 300, 40, moe(50, 4, 2))], 128, 64, {"start": 0, "stop": 1, "times": 2}, bigram=(3, 5, 2)),
+    # more heads than one workgroup takes, a latent past 128 seen from everywhere, more experts than most of the rows choose
+    "many": config([latent(18, 24, 20, 44, 130, 0, moe(40, 21, 5)), delta(6, 3, 100, 70, 4, dense(64)), latent(3, 70, 72, 36, 257, 150, None)], 132, 150, {"start": 1, "stop": 3, "times": 2},
+                   bigram=(67, 3, 11)),
     # one head, equal sizes, one pass
     "single": config([delta(1, 1, 128, 128, 4, dense(128)), latent(1, 128, 128, 128, 128, 128, moe(128, 2, 2))], 128, 128, {"start": 0, "stop": 2, "times": 1}, bigram=(128, 1, 1)),
 }
-RANKS = {"mixed": (18, 70), "odd": (7, 5), "plain": (64, 64), "wide": (130, 9), "single": (128, 128)}
+RANKS = {"mixed": (18, 70), "odd": (7, 5), "plain": (64, 64), "wide": (130, 9), "single": (128, 128), "many": (65, 30)}
 
 
 def steady_routing(cfg, w):
