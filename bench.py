@@ -971,7 +971,7 @@ def _vizosun_model(size, dev, dtype, max_position):
             shapes += [(p + f"mlp.e{e}.{n}", (W, EF) if n == "down" else (EF, W)) for e in range(E) for n in ("gate", "up", "down")]
         else:
             shapes += [(p + "mlp.gate", (F, W)), (p + "mlp.up", (F, W)), (p + "mlp.down", (W, F))]
-    c = VizosunConfig.from_dict({"vocab": V, "width": W, "layers": layers, "norm": {"eps": 1e-5}, "embedding": {"bigram": {"buckets": 8191, "mul_prev": 31, "mul_cur": 17}}, "loop": None}, dict(shapes))
+    c = VizosunConfig.from_dict({"vocab": V, "width": W, "layers": layers, "norm": {"eps": 1e-5}, "embedding": {"bigram": {"buckets": 8191, "mul_prev": 137, "mul_cur": 3}}, "loop": None}, dict(shapes))
     return _random_weights(VizosunForCausalLM(c, dtype=dtype, device=dev, max_position=max_position), shapes, dev, dtype)
 
 
